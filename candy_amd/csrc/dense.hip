@@ -1,0 +1,543 @@
+// bfloat16 weights [rows, cols]: upload, row gather and the contraction y = epilogue(x . W^T).
+//   k_dense_mv      one activation row: every weight row is streamed once by one wavefront, the activations wait in LDS
+//                   (bfloat16 or f32 activations; HBM-bound).  Optional prologue: the norms in front of the contraction.
+//   k_dense_mm      prompt batches, bfloat16 activations: v_mfma_f32_16x16x32_bf16 over LDS tiles filled by direct
+//                   global-to-LDS loads, two stages; optionally split along K
+//   k_dense_mm_f32  prompt batches, f32 activations: v_mfma_f32_16x16x4_f32, weights widened exactly
+// Weights are stored with both sides padded to multiples of 64 by zeros, so no kernel has a ragged edge in K, and the
+// padded rows come out as epilogue(0) = 0.  (No counterpart in the reference, which has no bfloat16.)
+#include <algorithm>
+
+#include "blocks.h"
+#include "dense.h"
+
+namespace candy {
+
+constexpr int EPI_NONE = CANDY_HIP_EPI_NONE, EPI_RELU2 = CANDY_HIP_EPI_SQUARED_RELU, EPI_CAP = CANDY_HIP_EPI_SOFTCAP;
+
+struct EpiArgs {
+    float scale, cap;
+};
+
+template <int EPI>
+__device__ __forceinline__ float epilogue(float z, const EpiArgs &e) {
+    if (EPI == EPI_RELU2) {
+        const float r = fmaxf(z, 0.0f);
+        return r * r;
+    }
+    if (EPI == EPI_CAP) {
+        z *= e.scale;
+        return e.cap > 0.0f ? e.cap * tanhf(z / e.cap) : z;
+    }
+    return z;
+}
+
+__device__ __forceinline__ void widen8(u32x4v v, float (&f)[8]) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        f[2 * i] = __uint_as_float(v[i] << 16);
+        f[2 * i + 1] = __uint_as_float(v[i] & 0xFFFF0000u);
+    }
+}
+__device__ __forceinline__ void lds8(const bf16 *p, float (&f)[8]) { widen8(*(const u32x4v *)p, f); }
+__device__ __forceinline__ void lds8(const float *p, float (&f)[8]) {
+    const f32x4 a = *(const f32x4 *)p, b = *(const f32x4 *)(p + 4);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) { f[i] = a[i]; f[4 + i] = b[i]; }
+}
+
+// ------------------------------------------------------------------ one row
+constexpr int MV_STEP = 2048;  // K values a wavefront takes per step: 4 x 64 lanes x 8
+
+template <class AT> constexpr int mv_lds_values() { return sizeof(AT) == 2 ? 16384 : 8192; }  // 32 KB: whole steps
+
+// R rows per wavefront; the next step's weights are requested before the current ones are multiplied, the first ones
+// before the activations are staged.
+template <class AT, int R, int EPI>
+__global__ __launch_bounds__(512) void k_dense_mv(const AT *__restrict__ x, const bf16 *__restrict__ W, void *__restrict__ yv,
+                                                  int K, int n_store, const EpiArgs ea) {
+    constexpr int U = 4, CH = mv_lds_values<AT>();
+    __shared__ __align__(16) AT xs[CH];
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const int row0 = (blockIdx.x * 8 + wave) * R;
+    const bf16 *wr = W + (size_t)row0 * K + lane * 8;
+    const int last = K - 8 - lane * 8;  // largest step offset this lane may load at
+    float acc[R];
+#pragma unroll
+    for (int r = 0; r < R; ++r) acc[r] = 0.0f;
+    auto fetch = [&](u32x4v (&w)[R][U], int k0) __attribute__((always_inline)) {
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+            const int k = max(min(k0 + u * 512, last), -lane * 8);  // past the row: any value of it, times x = 0
+#pragma unroll
+            for (int r = 0; r < R; ++r) w[r][u] = __builtin_nontemporal_load((const u32x4v *)(wr + (size_t)r * K + k));
+        }
+    };
+    auto multiply = [&](const u32x4v (&w)[R][U], int k0) __attribute__((always_inline)) {
+        const AT *xp = xs + (k0 & (CH - 1)) + lane * 8;
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+            float xf[8];
+            lds8(xp + u * 512, xf);
+#pragma unroll
+            for (int r = 0; r < R; ++r) {
+                float wf[8];
+                widen8(w[r][u], wf);
+#pragma unroll
+                for (int e = 0; e < 8; ++e) acc[r] = fmaf(wf[e], xf[e], acc[r]);
+            }
+        }
+    };
+    auto stage = [&](int k0) __attribute__((always_inline)) {
+        if (k0) __syncthreads();  // the previous chunk is consumed
+        const int n = min(CH, (K - k0 + MV_STEP - 1) / MV_STEP * MV_STEP);
+        constexpr int PER = 16 / sizeof(AT);
+        for (int i = tid * PER; i < n; i += 512 * PER)
+            *(u32x4v *)&xs[i] = k0 + i < K ? *(const u32x4v *)(x + k0 + i) : u32x4v{0, 0, 0, 0};
+        __syncthreads();
+    };
+    u32x4v wa[R][U], wb[R][U];
+    fetch(wa, 0);
+    for (int k0 = 0; k0 < K; k0 += 2 * MV_STEP) {
+        if ((k0 & (CH - 1)) == 0) stage(k0);
+        if (k0 + MV_STEP < K) fetch(wb, k0 + MV_STEP);
+        multiply(wa, k0);
+        if (k0 + MV_STEP >= K) break;
+        if (k0 + 2 * MV_STEP < K) fetch(wa, k0 + 2 * MV_STEP);
+        multiply(wb, k0 + MV_STEP);
+    }
+    float mine = 0.0f;
+#pragma unroll
+    for (int r = 0; r < R; ++r) {
+        const float t = wave_sum(acc[r]);
+        if (lane == r) mine = t;
+    }
+    if (lane < R && row0 + lane < n_store) {
+        const float z = epilogue<EPI>(mine, ea);
+        if (EPI == EPI_RELU2) ((AT *)yv)[row0 + lane] = (AT)z;
+        else ((float *)yv)[row0 + lane] = z;
+    }
+}
+
+// ------------------------------------------------------------------ prompt batches, bfloat16
+// Tile: BN = 128 weight rows x BM activation rows, 64 values of K per stage.  A row of a stage is 128 bytes = eight
+// 16-byte chunks; chunk c of row r sits in slot c ^ ((r >> 1) & 7), so that the 16 rows a fragment read touches spread
+// over all banks.  A direct load writes 64 consecutive 16-byte slots, so the permutation is in the addresses it reads.
+template <int BM, int EPI>
+__global__ __launch_bounds__(256, 2) void k_dense_mm(const bf16 *__restrict__ W, const bf16 *__restrict__ X, void *__restrict__ yv,
+                                                     int M, int Np, int ld, int ldx, int k_slice, int64_t ldy, int n_store,
+                                                     size_t split_stride, int m_tiles, int n_tiles, const EpiArgs ea) {
+    constexpr int BN = 128, BK = 64, ROWS = BN + BM, LOADS = ROWS / 32;
+    constexpr int TN = 4, TM = BM / 32;
+    __shared__ __align__(16) u32x4v s[2][ROWS * 8];
+    const int tid = threadIdx.x, lane = tid & 63;
+    const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    // each XCD takes a run of neighbouring tiles (workgroups are dealt to the XCDs round robin); the activation tiles of
+    // one weight tile are neighbours
+    const int total = m_tiles * n_tiles;
+    int t = blockIdx.x;
+    {
+        const int per = total >> 3, full = per << 3;
+        if (t < full) t = (t & 7) * per + (t >> 3);
+    }
+    const int m0 = (t % m_tiles) * BM, n0 = (t / m_tiles) * BN;
+    const int kbeg = blockIdx.y * k_slice, kend = min(kbeg + k_slice, ld);
+    const bf16 *src[LOADS];
+#pragma unroll
+    for (int i = 0; i < LOADS; ++i) {
+        const int r = (wave + 4 * i) * 8 + (lane >> 3);
+        const int c = (lane & 7) ^ ((r >> 1) & 7);
+        src[i] = (r < BN ? W + (size_t)min(n0 + r, Np - 1) * ld : X + (size_t)min(m0 + r - BN, M - 1) * ldx) + kbeg + c * 8;
+    }
+    auto load = [&](int stage) __attribute__((always_inline)) {
+#pragma unroll
+        for (int i = 0; i < LOADS; ++i) {
+            __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void *)src[i],
+                                             (__attribute__((address_space(3))) void *)&s[stage][(wave + 4 * i) * 64], 16, 0, 0);
+            src[i] += BK;
+        }
+    };
+    f32x4 acc[TN][TM];
+#pragma unroll
+    for (int i = 0; i < TN; ++i)
+#pragma unroll
+        for (int j = 0; j < TM; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+    const int wn = (wave >> 1) * 64, wm = BN + (wave & 1) * (BM / 2);
+    const int r16 = lane & 15, g = lane >> 4;
+    const int sw = (r16 >> 1) & 7;  // every tile starts at a multiple of 16 rows: the same swizzle for all of a lane's reads
+    auto compute = [&](int stage) __attribute__((always_inline)) {
+#pragma unroll
+        for (int kk = 0; kk < 2; ++kk) {
+            bf16x8 a[TN], b[TM];
+            const int slot = (kk * 4 + g) ^ sw;
+#pragma unroll
+            for (int i = 0; i < TN; ++i) a[i] = __builtin_bit_cast(bf16x8, s[stage][(wn + i * 16 + r16) * 8 + slot]);
+#pragma unroll
+            for (int j = 0; j < TM; ++j) b[j] = __builtin_bit_cast(bf16x8, s[stage][(wm + j * 16 + r16) * 8 + slot]);
+#pragma unroll
+            for (int i = 0; i < TN; ++i)
+#pragma unroll
+                for (int j = 0; j < TM; ++j) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[i], b[j], acc[i][j], 0, 0, 0);
+        }
+    };
+    const int n_it = (kend - kbeg) / BK;
+    load(0);
+    for (int it = 0; it < n_it; ++it) {
+        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+        __syncthreads();  // the stage has landed for every wavefront, and the other one is consumed
+        if (it + 1 < n_it) load((it + 1) & 1);
+        compute(it & 1);
+    }
+    // C layout: column r16 is the activation row, rows 4g .. 4g+3 are four neighbouring outputs of it
+#pragma unroll
+    for (int j = 0; j < TM; ++j) {
+        const int m = m0 + wm - BN + j * 16 + r16;
+        if (m >= M) continue;
+#pragma unroll
+        for (int i = 0; i < TN; ++i) {
+            const int n = n0 + wn + i * 16 + 4 * g;
+            f32x4 z = acc[i][j];
+#pragma unroll
+            for (int e = 0; e < 4; ++e) z[e] = epilogue<EPI>(z[e], ea);
+            if (EPI == EPI_RELU2) {
+                if (n < n_store) *(bf16x4 *)((bf16 *)yv + (size_t)m * ldy + n) = __builtin_convertvector(z, bf16x4);
+            } else if (EPI == EPI_NONE) {
+                float *y = (float *)yv + blockIdx.y * split_stride + (size_t)m * ldy + n;
+                if (n + 3 < n_store && (ldy & 3) == 0) *(f32x4 *)y = z;
+                else
+                    for (int e = 0; e < 4; ++e)
+                        if (n + e < n_store) y[e] = z[e];
+            } else {
+                float *y = (float *)yv + (size_t)m * ldy + n;
+#pragma unroll
+                for (int e = 0; e < 4; ++e)
+                    if (n + e < n_store) y[e] = z[e];
+            }
+        }
+    }
+}
+
+// ------------------------------------------------------------------ prompt batches, f32 activations
+template <int EPI>
+__global__ __launch_bounds__(256) void k_dense_mm_f32(const bf16 *__restrict__ W, const float *__restrict__ X, float *__restrict__ yv,
+                                                      int M, int ld, int ldx, int64_t ldy, int n_store, const EpiArgs ea) {
+    constexpr int B = 64, BK = 32, P = BK + 4;
+    __shared__ __align__(16) float sw[B * P], sx[B * P];
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const int n0 = blockIdx.x * B, m0 = blockIdx.y * B;
+    const int r16 = lane & 15, g = lane >> 4;
+    const int wn = (wave >> 1) * 32, wm = (wave & 1) * 32;
+    f32x4 acc[2][2];
+#pragma unroll
+    for (int i = 0; i < 2; ++i)
+#pragma unroll
+        for (int j = 0; j < 2; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+    const int lr = tid >> 2, lc = (tid & 3) * 8;  // a row of the stage, 8 of its 32 values
+    for (int k0 = 0; k0 < ld; k0 += BK) {
+        float wf[8], xf[8];
+        widen8(*(const u32x4v *)(W + (size_t)(n0 + lr) * ld + k0 + lc), wf);
+        lds8(X + (size_t)min(m0 + lr, M - 1) * ldx + k0 + lc, xf);
+        __syncthreads();
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+            sw[lr * P + lc + e] = wf[e];
+            sx[lr * P + lc + e] = xf[e];
+        }
+        __syncthreads();
+#pragma unroll
+        for (int kk = 0; kk < BK; kk += 4) {
+            float a[2], b[2];
+#pragma unroll
+            for (int i = 0; i < 2; ++i) {
+                a[i] = sw[(wn + i * 16 + r16) * P + kk + g];
+                b[i] = sx[(wm + i * 16 + r16) * P + kk + g];
+            }
+#pragma unroll
+            for (int i = 0; i < 2; ++i)
+#pragma unroll
+                for (int j = 0; j < 2; ++j) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x4f32(a[i], b[j], acc[i][j], 0, 0, 0);
+        }
+    }
+#pragma unroll
+    for (int j = 0; j < 2; ++j) {
+        const int m = m0 + wm + j * 16 + r16;
+        if (m >= M) continue;
+#pragma unroll
+        for (int i = 0; i < 2; ++i)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const int n = n0 + wn + i * 16 + 4 * g + e;
+                if (n < n_store) yv[(size_t)m * ldy + n] = epilogue<EPI>(acc[i][j][e], ea);
+            }
+    }
+}
+
+// ------------------------------------------------------------------ launches
+template <class AT, int R>
+static void launch_mv_epi(candy_hip_device *dev, const DenseLaunch &L) {
+    const dim3 g((unsigned)(L.w->rows_pad / (8 * R))), b(512);
+    const EpiArgs ea{L.scale, L.cap};
+    const AT *x = (const AT *)L.x;
+    const bf16 *W = (const bf16 *)L.w->data;
+    const int K = (int)L.w->ld, ns = (int)L.n_store;
+    switch (L.epi) {
+    case EPI_RELU2: hipLaunchKernelGGL((k_dense_mv<AT, R, EPI_RELU2>), g, b, 0, dev->stream, x, W, L.y, K, ns, ea); break;
+    case EPI_CAP: hipLaunchKernelGGL((k_dense_mv<AT, R, EPI_CAP>), g, b, 0, dev->stream, x, W, L.y, K, ns, ea); break;
+    default: hipLaunchKernelGGL((k_dense_mv<AT, R, EPI_NONE>), g, b, 0, dev->stream, x, W, L.y, K, ns, ea); break;
+    }
+}
+
+template <class AT>
+static int launch_mv(candy_hip_device *dev, const DenseLaunch &L) {
+    // enough wavefronts for eight per CU before rows are paired
+    const int64_t waves = 8 * (int64_t)dev->num_cus;
+    if (L.w->rows_pad >= 4 * waves) launch_mv_epi<AT, 4>(dev, L);
+    else if (L.w->rows_pad >= 2 * waves) launch_mv_epi<AT, 2>(dev, L);
+    else launch_mv_epi<AT, 1>(dev, L);
+    CANDY_LAUNCH_CHECK();
+    return CANDY_HIP_OK;
+}
+
+template <int BM>
+static int launch_mm(candy_hip_device *dev, const DenseLaunch &L) {
+    const int m_tiles = (L.m + BM - 1) / BM, n_tiles = (int)((L.w->rows_pad + 127) / 128);
+    const int64_t tiles = (int64_t)m_tiles * n_tiles;
+    CANDY_REQUIRE(tiles <= 0x7FFFFFFF, "matrix too large");
+    const int K = (int)L.w->ld;
+    int splits = 1;
+    void *y = L.y;
+    int64_t ldy = L.ldy, n_store = L.n_store;
+    size_t stride = 0;
+    if (L.partial) {
+        // two workgroups fit a CU; a slice keeps at least 512 values of K
+        const int64_t room = 2 * (int64_t)dev->num_cus / tiles;
+        splits = (int)std::max<int64_t>(1, std::min<int64_t>(std::min<int64_t>(room, 8), K / 512));
+        if (splits > 1) {
+            ldy = n_store = L.w->rows_pad;
+            stride = (size_t)L.m * ldy;
+            if (int rc = splitk_workspace(dev, stride * splits * sizeof(float), &y)) return rc;
+        }
+    }
+    const int k_slice = (int)pad64((K + splits - 1) / splits);
+    splits = (K + k_slice - 1) / k_slice;
+    if (L.partial) {
+        L.partial->p = (const float *)y;
+        L.partial->copies = splits;
+        L.partial->stride = stride;
+        L.partial->ld = (int)ldy;
+    }
+    const dim3 g((unsigned)tiles, (unsigned)splits), b(256);
+    const EpiArgs ea{L.scale, L.cap};
+    const bf16 *W = (const bf16 *)L.w->data, *X = (const bf16 *)L.x;
+#define CANDY_MM(EPI)                                                                                                     \
+    hipLaunchKernelGGL((k_dense_mm<BM, EPI>), g, b, 0, dev->stream, W, X, y, L.m, (int)L.w->rows_pad, K, (int)L.ldx, k_slice, \
+                       ldy, (int)n_store, stride, m_tiles, n_tiles, ea)
+    switch (L.epi) {
+    case EPI_RELU2: CANDY_MM(EPI_RELU2); break;
+    case EPI_CAP: CANDY_MM(EPI_CAP); break;
+    default: CANDY_MM(EPI_NONE); break;
+    }
+#undef CANDY_MM
+    CANDY_LAUNCH_CHECK();
+    return CANDY_HIP_OK;
+}
+
+int launch_dense(candy_hip_device *dev, const DenseLaunch &L) {
+    const candy_hip_dense *w = L.w;
+    CANDY_REQUIRE(L.m > 0 && w->rows_pad <= 0x7FFFFFFF && w->ld <= 0x7FFFFFFF && L.ldx >= w->ld && L.ldx <= 0x7FFFFFFF,
+                  "internal: dense contraction of a shape the kernels do not take");
+    CANDY_REQUIRE(L.n_store <= w->rows_pad && L.ldy >= L.n_store, "internal: dense output row too short");
+    CANDY_REQUIRE(L.epi != EPI_RELU2 || (L.n_store == w->rows_pad && (L.ldy & 63) == 0), "internal: activation rows must be padded");
+    if (L.partial) {
+        L.partial->p = (const float *)L.y;
+        L.partial->copies = 1;
+        L.partial->stride = 0;
+        L.partial->ld = (int)L.ldy;
+    }
+    if (L.m == 1) return L.f32 ? launch_mv<float>(dev, L) : launch_mv<bf16>(dev, L);
+    if (!L.f32) return L.m <= 64 ? launch_mm<64>(dev, L) : launch_mm<128>(dev, L);
+    const dim3 g((unsigned)(w->rows_pad / 64), (unsigned)((L.m + 63) / 64)), b(256);
+    CANDY_REQUIRE((L.m + 63) / 64 <= 65535, "prompt too long for one pass");
+    const EpiArgs ea{L.scale, L.cap};
+    const bf16 *W = (const bf16 *)w->data;
+    const float *X = (const float *)L.x;
+#define CANDY_MM32(EPI)                                                                                                 \
+    hipLaunchKernelGGL((k_dense_mm_f32<EPI>), g, b, 0, dev->stream, W, X, (float *)L.y, L.m, (int)w->ld, (int)L.ldx, L.ldy, \
+                       (int)L.n_store, ea)
+    switch (L.epi) {
+    case EPI_RELU2: CANDY_MM32(EPI_RELU2); break;
+    case EPI_CAP: CANDY_MM32(EPI_CAP); break;
+    default: CANDY_MM32(EPI_NONE); break;
+    }
+#undef CANDY_MM32
+    CANDY_LAUNCH_CHECK();
+    return CANDY_HIP_OK;
+}
+
+int launch_dense_norm(candy_hip_device *, const DenseLaunch &, const NormArgs &) { return CANDY_HIP_ERR_UNSUPPORTED; }
+
+// rows ids[i] of a bfloat16 table, widened; an id outside the table raises the handle's fault word and gives zeros
+__global__ __launch_bounds__(256) void k_dense_gather(const bf16 *__restrict__ W, int64_t rows, int64_t ld,
+                                                      const int64_t *__restrict__ ids, float *__restrict__ out, int64_t ldo,
+                                                      int *fault) {
+    const int64_t id = ids[blockIdx.y];
+    const int64_t c = ((int64_t)blockIdx.x * 256 + threadIdx.x) * 8;
+    if (c >= ld) return;
+    float f[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+    if (id >= 0 && id < rows) widen8(*(const u32x4v *)(W + id * ld + c), f);
+    else if (c == 0) *fault = 1;
+    float *o = out + (int64_t)blockIdx.y * ldo + c;
+    *(f32x4 *)o = f32x4{f[0], f[1], f[2], f[3]};
+    *(f32x4 *)(o + 4) = f32x4{f[4], f[5], f[6], f[7]};
+}
+
+int launch_dense_gather(candy_hip_device *dev, const candy_hip_dense *w, const int64_t *ids, int64_t n, float *out, int64_t ldo) {
+    for (int64_t i0 = 0; i0 < n; i0 += 65535) {
+        const int64_t part = std::min<int64_t>(n - i0, 65535);
+        hipLaunchKernelGGL(k_dense_gather, dim3((unsigned)((w->ld / 8 + 255) / 256), (unsigned)part), dim3(256), 0, dev->stream,
+                           (const bf16 *)w->data, w->rows, w->ld, ids + i0, out + i0 * ldo, ldo, dev->fault);
+        CANDY_LAUNCH_CHECK();
+    }
+    return CANDY_HIP_OK;
+}
+
+// f32 rows -> activation rows of ld values, zero past cols
+template <class AT>
+__global__ __launch_bounds__(256) void k_to_act(const float *__restrict__ src, AT *__restrict__ dst, int64_t rows, int64_t cols, int64_t ld) {
+    const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+    if (i >= rows * ld) return;
+    const int64_t r = i / ld, c = i % ld;
+    dst[i] = c < cols ? (AT)src[r * cols + c] : (AT)0.0f;
+}
+// activation rows -> dense f32
+template <class AT>
+__global__ __launch_bounds__(256) void k_from_act(const AT *__restrict__ src, float *__restrict__ dst, int64_t rows, int64_t cols, int64_t ld) {
+    const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+    if (i >= rows * cols) return;
+    dst[i] = (float)src[i / cols * ld + i % cols];
+}
+
+int launch_to_act(candy_hip_device *dev, bool f32, const float *src, void *dst, int64_t rows, int64_t cols, int64_t ld) {
+    const int64_t grid = (rows * ld + 255) / 256;
+    CANDY_REQUIRE(grid <= 0x7FFFFFFF, "matrix too large");
+    if (f32) hipLaunchKernelGGL((k_to_act<float>), dim3((unsigned)grid), dim3(256), 0, dev->stream, src, (float *)dst, rows, cols, ld);
+    else hipLaunchKernelGGL((k_to_act<bf16>), dim3((unsigned)grid), dim3(256), 0, dev->stream, src, (bf16 *)dst, rows, cols, ld);
+    CANDY_LAUNCH_CHECK();
+    return CANDY_HIP_OK;
+}
+int launch_from_act(candy_hip_device *dev, bool f32, const void *src, float *dst, int64_t rows, int64_t cols, int64_t ld) {
+    const int64_t grid = (rows * cols + 255) / 256;
+    CANDY_REQUIRE(grid <= 0x7FFFFFFF, "matrix too large");
+    if (f32) hipLaunchKernelGGL((k_from_act<float>), dim3((unsigned)grid), dim3(256), 0, dev->stream, (const float *)src, dst, rows, cols, ld);
+    else hipLaunchKernelGGL((k_from_act<bf16>), dim3((unsigned)grid), dim3(256), 0, dev->stream, (const bf16 *)src, dst, rows, cols, ld);
+    CANDY_LAUNCH_CHECK();
+    return CANDY_HIP_OK;
+}
+
+}  // namespace candy
+
+using namespace candy;
+
+extern "C" {
+
+int candy_hip_dense_upload(candy_hip_device *dev, int64_t rows, int64_t cols, const uint16_t *host_bf16, candy_hip_dense **out) {
+    CANDY_REQUIRE(out, "out is nil");
+    *out = nullptr;
+    CANDY_REQUIRE(dev, "device handle is nil");
+    CANDY_REQUIRE(rows > 0 && cols > 0 && rows <= 0x7FFFFF00 && cols <= 0x7FFFFF00, "invalid matrix dimensions %lld x %lld",
+                  (long long)rows, (long long)cols);
+    CANDY_REQUIRE(host_bf16, "host weight is nil");
+    if (int rc = use_device(dev)) return rc;
+    const int64_t rp = pad64(rows), ld = pad64(cols);
+    void *d = nullptr;
+    const size_t bytes = (size_t)rp * ld * 2;
+    if (int rc = candy_hip_alloc(dev, bytes, &d)) return rc;
+    int rc = CANDY_HIP_OK;
+    if (rp != rows || ld != cols) rc = candy_hip_zero(dev, d, bytes);
+    if (!rc) {
+        hipError_t e = hipMemcpy2DAsync(d, (size_t)ld * 2, host_bf16, (size_t)cols * 2, (size_t)cols * 2, (size_t)rows,
+                                        hipMemcpyHostToDevice, dev->stream);
+        if (e == hipSuccess) e = hipStreamSynchronize(dev->stream);
+        if (e != hipSuccess) rc = fail(CANDY_HIP_ERR_HIP, "weight upload failed: %s", hipGetErrorString(e));
+    }
+    if (rc) {
+        (void)candy_hip_free(dev, d);
+        return rc;
+    }
+    candy_hip_dense *w = new candy_hip_dense();
+    w->dev = dev; w->rows = rows; w->cols = cols; w->rows_pad = rp; w->ld = ld; w->data = d;
+    *out = w;
+    return CANDY_HIP_OK;
+}
+
+int candy_hip_dense_free(candy_hip_dense *w) {
+    if (!w) return CANDY_HIP_OK;
+    const int rc = candy_hip_free(w->dev, w->data);
+    delete w;
+    return rc;
+}
+
+int candy_hip_dense_info(const candy_hip_dense *w, int64_t *rows, int64_t *cols, size_t *nbytes) {
+    CANDY_REQUIRE(w, "weight is nil");
+    if (rows) *rows = w->rows;
+    if (cols) *cols = w->cols;
+    if (nbytes) *nbytes = (size_t)w->rows_pad * w->ld * 2;
+    return CANDY_HIP_OK;
+}
+
+int candy_hip_dense_matmul(candy_hip_device *dev, const candy_hip_dense *w, const float *dev_x, int64_t m, int act, int epilogue,
+                           float scale, float cap, float *dev_y) {
+    CANDY_REQUIRE(w, "rhs weight is nil");
+    CANDY_REQUIRE(dev && w->dev == dev, "rhs storage must live on the same HIP device");
+    CANDY_REQUIRE(m >= 0 && m <= 1 << 20, "invalid matrix dimensions");
+    CANDY_REQUIRE(act == CANDY_HIP_ACT_BF16 || act == CANDY_HIP_ACT_F32, "unknown activation format %d", act);
+    CANDY_REQUIRE(epilogue >= EPI_NONE && epilogue <= EPI_CAP, "unknown epilogue %d", epilogue);
+    if (m == 0) return CANDY_HIP_OK;
+    CANDY_REQUIRE(dev_x && dev_y, "nil pointer");
+    if (int rc = use_device(dev)) return rc;
+    const bool f32 = act == CANDY_HIP_ACT_F32;
+    const size_t x_bytes = (size_t)m * w->ld * 4, y_bytes = (size_t)m * w->rows_pad * 4;
+    void *ws = nullptr;
+    if (int rc = workspace(dev, x_bytes + y_bytes, &ws)) return rc;
+    if (int rc = launch_to_act(dev, f32, dev_x, ws, m, w->cols, w->ld)) return rc;
+    DenseLaunch L;
+    L.w = w; L.x = ws; L.ldx = w->ld; L.f32 = f32; L.m = (int)m; L.epi = epilogue; L.scale = scale; L.cap = cap;
+    if (epilogue != EPI_RELU2) {
+        L.y = dev_y; L.ldy = L.n_store = w->rows;
+        return launch_dense(dev, L);
+    }
+    L.y = (uint8_t *)ws + x_bytes; L.ldy = L.n_store = w->rows_pad;
+    if (int rc = launch_dense(dev, L)) return rc;
+    return launch_from_act(dev, f32, L.y, dev_y, m, w->rows, w->rows_pad);
+}
+
+int candy_hip_dense_sweep(candy_hip_device *dev, const candy_hip_dense *const *ws, int n_ws, const float *dev_x, int64_t m,
+                          int epilogue, int iters, float *elapsed_ms) {
+    CANDY_REQUIRE(dev && ws && n_ws > 0 && dev_x && elapsed_ms && iters > 0 && m > 0 && m <= 1 << 20, "nil argument");
+    CANDY_REQUIRE(epilogue >= EPI_NONE && epilogue <= EPI_CAP, "unknown epilogue %d", epilogue);
+    for (int i = 0; i < n_ws; ++i)
+        CANDY_REQUIRE(ws[i] && ws[i]->dev == dev && ws[i]->rows == ws[0]->rows && ws[i]->cols == ws[0]->cols,
+                      "weights of one sweep share a device and a shape");
+    if (int rc = use_device(dev)) return rc;
+    const candy_hip_dense *w = ws[0];
+    const size_t x_bytes = (size_t)m * w->ld * 2;
+    void *buf = nullptr;
+    if (int rc = workspace(dev, x_bytes + (size_t)m * w->rows_pad * 4, &buf)) return rc;
+    if (int rc = launch_to_act(dev, false, dev_x, buf, m, w->cols, w->ld)) return rc;
+    DenseLaunch L;
+    Partial part;
+    L.x = buf; L.ldx = w->ld; L.m = (int)m; L.epi = epilogue; L.scale = 1.0f; L.cap = 30.0f;
+    L.y = (uint8_t *)buf + x_bytes; L.ldy = L.n_store = w->rows_pad;
+    if (epilogue == EPI_NONE) L.partial = &part;
+    CANDY_HIP_TRY(hipEventRecord(dev->ev_start, dev->stream));
+    for (int i = 0; i < iters; ++i) {
+        L.w = ws[i % n_ws];
+        if (int rc = launch_dense(dev, L)) return rc;
+    }
+    CANDY_HIP_TRY(hipEventRecord(dev->ev_stop, dev->stream));
+    CANDY_HIP_TRY(hipEventSynchronize(dev->ev_stop));
+    CANDY_HIP_TRY(hipEventElapsedTime(elapsed_ms, dev->ev_start, dev->ev_stop));
+    return CANDY_HIP_OK;
+}
+
+}  // extern "C"

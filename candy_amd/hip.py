@@ -8,7 +8,7 @@ from __future__ import annotations
 
 import ctypes
 import os
-from ctypes import POINTER, byref, c_char_p, c_float, c_int, c_int32, c_int64, c_size_t, c_uint32, c_void_p
+from ctypes import POINTER, byref, c_char_p, c_double, c_float, c_int, c_int32, c_int64, c_size_t, c_uint32, c_void_p
 
 import numpy as np
 
@@ -32,6 +32,28 @@ class LlamaConfig(ctypes.Structure):
                 ("head_dim", c_int32), ("d_ffn", c_int32), ("vocab", c_int32), ("max_pos", c_int32),
                 ("rms_eps", c_float), ("rope_base", c_float)]
 
+
+class AttnSpec(ctypes.Structure):
+    _fields_ = [("n_heads", c_int32), ("n_kv_heads", c_int32), ("head_dim", c_int32), ("window", c_int32),
+                ("rope_dims", c_int32), ("rope_original", c_int32), ("scale", c_float), ("softcap", c_float),
+                ("rope_base", c_double), ("rope_factor", c_double), ("rope_low", c_double), ("rope_high", c_double)]
+
+
+class SuvazenLayer(ctypes.Structure):
+    _fields_ = [("attn", AttnSpec), ("d_ffn", c_int32), ("has_sink", c_int32)]
+
+
+class SuvazenConfig(ctypes.Structure):
+    _fields_ = [("n_layers", c_int32), ("d_model", c_int32), ("vocab", c_int32), ("max_pos", c_int32),
+                ("loop_start", c_int32), ("loop_stop", c_int32), ("loop_times", c_int32), ("act", c_int32),
+                ("norm_eps", c_float), ("residual_mult", c_float), ("logit_scale", c_float), ("logit_softcap", c_float)]
+
+
+ACT_BF16, ACT_F32 = 0, 1
+EPI_NONE, EPI_SQUARED_RELU, EPI_SOFTCAP = 0, 1, 2
+SV_QK, SV_O, SV_UP, SV_DOWN, SV_HEAD, SV_EMBED = range(6)
+(SV_NORM1, SV_NORM1_BIAS, SV_NORM1B, SV_NORM1B_BIAS, SV_NORM2, SV_NORM2_BIAS, SV_NORM2B, SV_NORM2B_BIAS, SV_SINK, SV_STEP,
+ SV_FINAL, SV_FINAL_BIAS) = range(12)
 
 # name -> (restype, argtypes); exactly the symbols include/candy_hip.h declares
 SIGNATURES = {
@@ -105,6 +127,33 @@ SIGNATURES = {
     "candy_hip_llama_decode_hidden": (c_int, [c_void_p, c_void_p, c_int32, POINTER(c_void_p), POINTER(c_int32)]),
     "candy_hip_llama_prefill": (c_int, [c_void_p, POINTER(c_int32), c_int32, c_int32, POINTER(c_void_p),
                                         POINTER(c_int32)]),
+    "candy_hip_llama_decoder": (c_void_p, [c_void_p]),
+    "candy_hip_dense_upload": (c_int, [c_void_p, c_int64, c_int64, c_void_p, POINTER(c_void_p)]),
+    "candy_hip_dense_free": (c_int, [c_void_p]),
+    "candy_hip_dense_info": (c_int, [c_void_p, POINTER(c_int64), POINTER(c_int64), POINTER(c_size_t)]),
+    "candy_hip_dense_matmul": (c_int, [c_void_p, c_void_p, c_void_p, c_int64, c_int, c_int, c_float, c_float, c_void_p]),
+    "candy_hip_dense_sweep": (c_int, [c_void_p, POINTER(c_void_p), c_int, c_void_p, c_int64, c_int, c_int, POINTER(c_float)]),
+    "candy_hip_layer_norm": (c_int, [c_void_p, c_void_p, c_void_p, c_void_p, c_float, c_int64, c_int64, c_void_p]),
+    "candy_hip_add_layer_norm": (c_int, [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_float, c_float, c_void_p,
+                                         c_int64, c_int64]),
+    "candy_hip_attn_row": (c_int, [c_int]),
+    "candy_hip_window_attention": (c_int, [c_void_p, POINTER(AttnSpec), c_int, c_void_p, c_int64, c_int32, c_int32, c_void_p,
+                                           c_void_p, c_void_p, c_int, c_void_p]),
+    "candy_hip_decoder_free": (c_int, [c_void_p]),
+    "candy_hip_decoder_set_graph": (c_int, [c_void_p, c_int]),
+    "candy_hip_decoder_hidden": (c_int, [c_void_p, POINTER(c_void_p)]),
+    "candy_hip_decoder_kv_cache": (c_int, [c_void_p, POINTER(c_void_p), POINTER(c_void_p), POINTER(c_size_t)]),
+    "candy_hip_decoder_decode": (c_int, [c_void_p, c_int32, c_int32, POINTER(c_void_p), POINTER(c_int32)]),
+    "candy_hip_decoder_decode_hidden": (c_int, [c_void_p, c_void_p, c_int32, POINTER(c_void_p), POINTER(c_int32)]),
+    "candy_hip_decoder_generate": (c_int, [c_void_p, c_int32, c_int32, c_int32, POINTER(c_int32)]),
+    "candy_hip_decoder_prefill": (c_int, [c_void_p, POINTER(c_int32), c_int32, c_int32, POINTER(c_void_p), POINTER(c_int32)]),
+    "candy_hip_decoder_prefill_rows": (c_int, [c_void_p, POINTER(c_int32), c_int32, c_int32, POINTER(c_int32), c_int32,
+                                               POINTER(c_void_p)]),
+    "candy_hip_decoder_prompt_hidden": (c_int, [c_void_p, POINTER(c_void_p), POINTER(c_int64)]),
+    "candy_hip_suvazen_create": (c_int, [c_void_p, POINTER(SuvazenConfig), POINTER(SuvazenLayer), POINTER(c_void_p)]),
+    "candy_hip_suvazen_decoder": (c_void_p, [c_void_p]),
+    "candy_hip_suvazen_set_matrix": (c_int, [c_void_p, c_int, c_int, c_void_p]),
+    "candy_hip_suvazen_set_vector": (c_int, [c_void_p, c_int, c_int, c_void_p, c_int64]),
     "candy_hip_qmatmul_sweep": (c_int, [c_void_p, POINTER(c_void_p), c_int, c_void_p, c_int64, c_void_p, c_int, c_int,
                                         POINTER(c_float)]),
     "candy_hip_qmatmul_sustained_sweep": (c_int, [c_void_p, POINTER(c_void_p), c_int, c_int, c_int, c_void_p, c_void_p, c_int,
@@ -215,6 +264,46 @@ class QTensor:
     def free(self):
         if self.handle is not None and self.dev.handle is not None:
             _check(lib().candy_hip_qtensor_free(self.handle))
+        self.handle = None
+
+    def __del__(self):
+        try:
+            self.free()
+        except Exception:
+            pass
+
+
+def bf16_bits(x: np.ndarray) -> np.ndarray:
+    """float32 -> bfloat16 bit patterns, rounded to nearest even (finite inputs)."""
+    u = np.ascontiguousarray(x, np.float32).view(np.uint32)
+    return ((u + 0x7FFF + ((u >> 16) & 1)) >> 16).astype(np.uint16)
+
+
+def bf16_values(bits: np.ndarray) -> np.ndarray:
+    """bfloat16 bit patterns -> float32."""
+    return (np.ascontiguousarray(bits, np.uint16).astype(np.uint32) << 16).view(np.float32)
+
+
+class Dense:
+    """Device-resident bfloat16 weight [rows, cols]; `bits` are the raw 16-bit values."""
+
+    def __init__(self, dev: "Device", bits: np.ndarray):
+        b = np.ascontiguousarray(bits)
+        if b.dtype != np.uint16 or b.ndim != 2:
+            raise ValueError("a dense weight is a 2-D array of bfloat16 bit patterns (uint16)")
+        h = c_void_p()
+        _check(lib().candy_hip_dense_upload(dev.handle, b.shape[0], b.shape[1], b.ctypes.data, byref(h)))
+        self.dev, self.rows, self.cols, self.handle = dev, b.shape[0], b.shape[1], h.value
+
+    @property
+    def nbytes(self) -> int:
+        n = c_size_t()
+        _check(lib().candy_hip_dense_info(self.handle, None, None, byref(n)))
+        return n.value
+
+    def free(self):
+        if self.handle is not None and self.dev.handle is not None:
+            _check(lib().candy_hip_dense_free(self.handle))
         self.handle = None
 
     def __del__(self):
@@ -458,6 +547,58 @@ class Device:
                                                 n_pos, cache_stride, scale, out.ptr))
         return out.download(np.float32, n_heads * head_dim)
 
+    # ---- bfloat16 weights, layer norms, windowed attention
+    def dense(self, bits: np.ndarray) -> Dense:
+        return Dense(self, bits)
+
+    def dense_matmul(self, w: Dense, x, act: int = ACT_BF16, epilogue: int = EPI_NONE, scale: float = 1.0,
+                     cap: float = 0.0) -> np.ndarray:
+        x = np.ascontiguousarray(x, np.float32).reshape(-1, w.cols)
+        m = x.shape[0]
+        src, dst = self.from_numpy(x), self.alloc(max(m * w.rows * 4, 4))
+        _check(lib().candy_hip_dense_matmul(self.handle, w.handle, src.ptr, m, act, epilogue, scale, cap, dst.ptr))
+        return dst.download(np.float32, m * w.rows).reshape(m, w.rows)
+
+    def dense_sweep(self, weights: list, x_buf: "Buffer", m: int, iters: int, epilogue: int = EPI_NONE) -> float:
+        """Elapsed milliseconds of `iters` back-to-back bfloat16 contractions rotating over `weights`."""
+        arr = (c_void_p * len(weights))(*[w.handle for w in weights])
+        ms = c_float(0)
+        _check(lib().candy_hip_dense_sweep(self.handle, arr, len(weights), x_buf.ptr, m, epilogue, iters, byref(ms)))
+        return ms.value
+
+    def layer_norm(self, x, w, b, eps: float) -> np.ndarray:
+        x = np.ascontiguousarray(x, np.float32)
+        cols = x.shape[-1]
+        dx, dw, db, out = self._f32(x), self._f32(w), self._f32(b), self.alloc(max(x.nbytes, 4))
+        _check(lib().candy_hip_layer_norm(self.handle, dx.ptr, dw.ptr, db.ptr, eps, x.size // cols, cols, out.ptr))
+        return out.download(np.float32, x.size).reshape(x.shape)
+
+    def add_layer_norm(self, x, y, w, b, eps: float, mult: float, step=None) -> np.ndarray:
+        """x + mult * layer_norm(y) (+ step)"""
+        x = np.ascontiguousarray(x, np.float32)
+        cols = x.shape[-1]
+        dx, dy, dw, db = self._f32(x), self._f32(y), self._f32(w), self._f32(b)
+        ds = self._f32(step) if step is not None else None
+        _check(lib().candy_hip_add_layer_norm(self.handle, dx.ptr, dy.ptr, dw.ptr, db.ptr, eps, mult,
+                                              ds.ptr if ds else None, x.size // cols, cols))
+        return dx.download(np.float32, x.size).reshape(x.shape)
+
+    def window_attention(self, spec: AttnSpec, act: int, qk, pos0: int, max_pos: int, k_cache: "Buffer", v_cache: "Buffer",
+                         sink=None, decode: bool = False) -> np.ndarray:
+        """qk [n, (n_heads + n_kv_heads) * head_dim] at positions pos0 ..; the caches receive the new rows."""
+        qk = np.ascontiguousarray(qk, np.float32)
+        n, width = qk.shape[0], spec.n_heads * spec.head_dim
+        if qk.shape[1] != width + spec.n_kv_heads * spec.head_dim:
+            raise ValueError("qk rows do not fit the spec")
+        need = spec.n_kv_heads * max_pos * lib().candy_hip_attn_row(spec.head_dim) * (4 if act == ACT_F32 else 2)
+        if k_cache.nbytes < need or v_cache.nbytes < need:
+            raise ValueError("cache too small")
+        dq, out = self._f32(qk), self.alloc(n * width * 4)
+        ds = self._f32(sink) if sink is not None else None
+        _check(lib().candy_hip_window_attention(self.handle, byref(spec), act, dq.ptr, n, pos0, max_pos, k_cache.ptr,
+                                                v_cache.ptr, ds.ptr if ds else None, int(decode), out.ptr))
+        return out.download(np.float32, n * width).reshape(n, width)
+
     # ---- timing
     def qmatmul_sweep(self, weights: list, x_buf: "Buffer", m: int, y_buf: "Buffer", iters: int,
                       quantize_each: bool = True) -> float:
@@ -514,20 +655,16 @@ class Device:
         return ms.value
 
 
-class Llama:
-    """Llama-style decoder on the device (weights stay owned by the caller)."""
+class Decoder:
+    """Any decoder of the library: one sequence in its cache, fed token by token or in portions.
 
-    def __init__(self, dev: Device, **cfg):
-        self.dev = dev
-        self.cfg = LlamaConfig(**cfg)
-        h = c_void_p()
-        _check(lib().candy_hip_llama_create(dev.handle, byref(self.cfg), byref(h)))
-        self.handle = h.value
-        self._keep = []
+    Subclasses create the model and set `self.handle` to its decoder handle, `self.width`, `self.vocab`, `self.max_pos`."""
+
+    handle = None
 
     def free(self):
         if self.handle is not None and self.dev.handle is not None:
-            _check(lib().candy_hip_llama_free(self.handle))
+            _check(lib().candy_hip_decoder_free(self.handle))
         self.handle = None
 
     def __del__(self):
@@ -536,62 +673,124 @@ class Llama:
         except Exception:
             pass
 
-    def set_qweight(self, which: int, layer: int, w: QTensor):
-        self._keep.append(w)
-        _check(lib().candy_hip_llama_set_qweight(self.handle, which, layer, w.handle))
-
-    def set_norm(self, which: int, layer: int, alpha: np.ndarray):
-        buf = self.dev.from_numpy(np.ascontiguousarray(alpha, np.float32))
-        self._keep.append(buf)
-        _check(lib().candy_hip_llama_set_norm(self.handle, which, layer, buf.ptr))
-
     def set_graph(self, enable: bool):
-        _check(lib().candy_hip_llama_set_graph(self.handle, int(enable)))
-
-    def set_kv_f16(self, enable: bool):
-        """fp16 KV cache (clears the cache); kv_cache() then reports half the bytes."""
-        _check(lib().candy_hip_llama_set_kv_f16(self.handle, int(enable)))
+        _check(lib().candy_hip_decoder_set_graph(self.handle, int(enable)))
 
     def kv_cache(self):
         k, v, n = c_void_p(), c_void_p(), c_size_t()
-        _check(lib().candy_hip_llama_kv_cache(self.handle, byref(k), byref(v), byref(n)))
+        _check(lib().candy_hip_decoder_kv_cache(self.handle, byref(k), byref(v), byref(n)))
         return k.value, v.value, n.value
 
     def hidden(self) -> np.ndarray:
         """The residual stream as the last decode step left it behind the last layer (before the final norm)."""
         p = c_void_p()
-        _check(lib().candy_hip_llama_hidden(self.handle, byref(p)))
-        out = np.empty(self.cfg.d_model, np.float32)
-        _check(lib().candy_hip_d2h(self.dev.handle, out.ctypes.data, p.value, out.nbytes))
-        return out
+        _check(lib().candy_hip_decoder_hidden(self.handle, byref(p)))
+        return self._download(p.value, self.width)
+
+    def prompt_hidden(self, n_tokens: int) -> np.ndarray:
+        """The residual stream of the last prompt pass's first n_tokens tokens behind the last layer."""
+        p, ld = c_void_p(), c_int64()
+        _check(lib().candy_hip_decoder_prompt_hidden(self.handle, byref(p), byref(ld)))
+        return self._download(p.value, n_tokens * ld.value).reshape(n_tokens, ld.value)[:, :self.width].copy()
 
     def decode(self, token: int, pos: int, want_logits: bool = True):
         lg, nt = c_void_p(), c_int32(-1)
-        _check(lib().candy_hip_llama_decode(self.handle, token, pos, byref(lg), byref(nt)))
-        return self._result(lg, nt, want_logits)
+        _check(lib().candy_hip_decoder_decode(self.handle, token, pos, byref(lg), byref(nt)))
+        return nt.value, self._download(lg.value, self.vocab) if want_logits else None
 
     def generate(self, token: int, pos: int, n_steps: int):
         """n_steps greedy steps without a host round trip between them; returns the chosen tokens."""
         out = (c_int32 * n_steps)()
-        _check(lib().candy_hip_llama_generate(self.handle, token, pos, n_steps, out))
+        _check(lib().candy_hip_decoder_generate(self.handle, token, pos, n_steps, out))
         return [int(t) for t in out]
 
     def decode_hidden(self, hidden: np.ndarray, pos: int, want_logits: bool = True):
         buf = self.dev.from_numpy(np.ascontiguousarray(hidden, np.float32))
         lg, nt = c_void_p(), c_int32(-1)
-        _check(lib().candy_hip_llama_decode_hidden(self.handle, buf.ptr, pos, byref(lg), byref(nt)))
-        return self._result(lg, nt, want_logits)
+        _check(lib().candy_hip_decoder_decode_hidden(self.handle, buf.ptr, pos, byref(lg), byref(nt)))
+        return nt.value, self._download(lg.value, self.vocab) if want_logits else None
 
     def prefill(self, tokens, pos0: int = 0, want_logits: bool = True):
         """Batched prompt pass; returns (greedy next token, logits) of the last prompt token."""
         ids = (c_int32 * len(tokens))(*[int(t) for t in tokens])
         lg, nt = c_void_p(), c_int32(-1)
-        _check(lib().candy_hip_llama_prefill(self.handle, ids, len(tokens), pos0, byref(lg), byref(nt)))
-        return self._result(lg, nt, want_logits)
+        _check(lib().candy_hip_decoder_prefill(self.handle, ids, len(tokens), pos0, byref(lg), byref(nt)))
+        return nt.value, self._download(lg.value, self.vocab) if want_logits else None
 
-    def _result(self, lg, nt, want_logits):
-        logits = None
-        if want_logits:
-            logits = np.empty(self.cfg.vocab, np.float32)
-            _check(lib().candy_hip_d2h(self.dev.handle, logits.ctypes.data, lg.value, logits.nbytes))
-        return nt.value, logits
+    def feed(self, tokens, pos0: int = 0, want=()) -> np.ndarray:
+        """The next tokens of the sequence, at positions pos0 ..; logits [len(want), vocab] of the chosen ones (counted
+        from the first of `tokens`).  One token takes the decode step, more take the prompt pass."""
+        want = [int(w) for w in want]
+        if any(w < 0 or w >= len(tokens) for w in want):
+            raise ValueError("a wanted place lies outside the tokens fed")
+        if len(tokens) == 1:
+            lg = c_void_p()
+            _check(lib().candy_hip_decoder_decode(self.handle, int(tokens[0]), pos0, byref(lg), None))
+            if not want:
+                return np.empty((0, self.vocab), np.float32)
+            return np.tile(self._download(lg.value, self.vocab), (len(want), 1))
+        ids = (c_int32 * len(tokens))(*[int(t) for t in tokens])
+        rows = (c_int32 * max(len(want), 1))(*want)
+        lg = c_void_p()
+        _check(lib().candy_hip_decoder_prefill_rows(self.handle, ids, len(tokens), pos0, rows, len(want), byref(lg)))
+        return self._download(lg.value, len(want) * self.vocab).reshape(len(want), self.vocab) if want \
+            else np.empty((0, self.vocab), np.float32)
+
+    def greedy(self, prompt, n_steps: int):
+        """The n_steps tokens greedy decoding appends to a prompt."""
+        tok, _ = self.prefill(prompt, 0, want_logits=False)
+        return [tok] + (self.generate(tok, len(prompt), n_steps - 1) if n_steps > 1 else [])
+
+    def _download(self, ptr: int, count: int) -> np.ndarray:
+        out = np.empty(count, np.float32)
+        _check(lib().candy_hip_d2h(self.dev.handle, out.ctypes.data, ptr, out.nbytes))
+        return out
+
+
+class Llama(Decoder):
+    """Llama-style decoder on the device (weights stay owned by the caller)."""
+
+    def __init__(self, dev: Device, **cfg):
+        self.dev = dev
+        self.cfg = LlamaConfig(**cfg)
+        h = c_void_p()
+        _check(lib().candy_hip_llama_create(dev.handle, byref(self.cfg), byref(h)))
+        self.model = h.value
+        self.handle = lib().candy_hip_llama_decoder(self.model)
+        self.width, self.vocab, self.max_pos = self.cfg.d_model, self.cfg.vocab, self.cfg.max_pos
+        self._keep = []
+
+    def set_qweight(self, which: int, layer: int, w: QTensor):
+        self._keep.append(w)
+        _check(lib().candy_hip_llama_set_qweight(self.model, which, layer, w.handle))
+
+    def set_norm(self, which: int, layer: int, alpha: np.ndarray):
+        buf = self.dev.from_numpy(np.ascontiguousarray(alpha, np.float32))
+        self._keep.append(buf)
+        _check(lib().candy_hip_llama_set_norm(self.model, which, layer, buf.ptr))
+
+    def set_kv_f16(self, enable: bool):
+        """fp16 KV cache (clears the cache); kv_cache() then reports half the bytes."""
+        _check(lib().candy_hip_llama_set_kv_f16(self.model, int(enable)))
+
+
+class Suvazen(Decoder):
+    """Suvazen decoder on the device (candy_amd/suvazen.py builds one from a model folder)."""
+
+    def __init__(self, dev: Device, cfg: SuvazenConfig, layers: list):
+        self.dev, self.cfg = dev, cfg
+        self.layers = (SuvazenLayer * len(layers))(*layers)
+        h = c_void_p()
+        _check(lib().candy_hip_suvazen_create(dev.handle, byref(cfg), self.layers, byref(h)))
+        self.model = h.value
+        self.handle = lib().candy_hip_suvazen_decoder(self.model)
+        self.width, self.vocab, self.max_pos = cfg.d_model, cfg.vocab, cfg.max_pos
+        self._keep = []
+
+    def set_matrix(self, which: int, layer: int, w: Dense):
+        self._keep.append(w)
+        _check(lib().candy_hip_suvazen_set_matrix(self.model, which, layer, w.handle))
+
+    def set_vector(self, which: int, layer: int, values: np.ndarray):
+        v = np.ascontiguousarray(values, np.float32).reshape(-1)
+        _check(lib().candy_hip_suvazen_set_vector(self.model, which, layer, v.ctypes.data, v.size))

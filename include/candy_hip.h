@@ -28,6 +28,8 @@ extern "C" {
 typedef struct candy_hip_device candy_hip_device;     /* one GPU + its stream + its workspace   */
 typedef struct candy_hip_qtensor candy_hip_qtensor;   /* device-resident quantized weight matrix */
 typedef struct candy_hip_qact candy_hip_qact;         /* activations quantized once, reusable     */
+typedef struct candy_hip_dense candy_hip_dense;       /* device-resident bfloat16 weight matrix    */
+typedef struct candy_hip_decoder candy_hip_decoder;   /* any decoder: cache, step, prompt, generation */
 typedef struct candy_hip_llama candy_hip_llama;       /* Llama-style decoder built on the ops    */
 
 enum candy_hip_status {
@@ -357,6 +359,126 @@ int candy_hip_llama_decode_hidden(candy_hip_llama *m, const float *dev_hidden, i
  * to n_tokens successive candy_hip_llama_decode calls up to f32 summation order. */
 int candy_hip_llama_prefill(candy_hip_llama *m, const int32_t *tokens, int32_t n_tokens, int32_t pos0,
                             const float **dev_logits, int32_t *next_token);
+
+/* The decoder behind the handle (the same object; freed with candy_hip_llama_free or candy_hip_decoder_free). */
+candy_hip_decoder *candy_hip_llama_decoder(candy_hip_llama *m);
+
+/* ------------------------------------------------------------------ bfloat16 weights and the ops around them
+ * No counterpart in the reference (candy.D has no bfloat16; dtype.go:4-6).  A dense weight is row-major [rows, cols]
+ * bfloat16 on the host (raw 16-bit values); the device copy pads both sides with zeros to multiples of 64. */
+int candy_hip_dense_upload(candy_hip_device *dev, int64_t rows, int64_t cols, const uint16_t *host_bf16,
+                           candy_hip_dense **out);
+int candy_hip_dense_free(candy_hip_dense *w);
+int candy_hip_dense_info(const candy_hip_dense *w, int64_t *rows, int64_t *cols, size_t *nbytes);
+
+/* Number format of the activations a dense weight is contracted with.  BF16: activations rounded to bfloat16, products
+ * accumulated in f32 (matrix cores from two rows up).  F32: activations and sums in f32, the weights' bfloat16 values
+ * widened exactly. */
+enum candy_hip_act { CANDY_HIP_ACT_BF16 = 0, CANDY_HIP_ACT_F32 = 1 };
+/* What follows the contraction z: NONE z; SQUARED_RELU max(z, 0)^2; SOFTCAP cap * tanh(scale * z / cap), or scale * z
+ * with cap 0. */
+enum candy_hip_epilogue { CANDY_HIP_EPI_NONE = 0, CANDY_HIP_EPI_SQUARED_RELU = 1, CANDY_HIP_EPI_SOFTCAP = 2 };
+/* y[m, rows] = epilogue(x[m, cols] . W^T), f32 in and out (x is converted on the device where act asks for it; the
+ * squared ReLU's output is rounded to the activation format, as the next contraction reads it). */
+int candy_hip_dense_matmul(candy_hip_device *dev, const candy_hip_dense *w, const float *dev_x, int64_t m, int act,
+                           int epilogue, float scale, float cap, float *dev_y);
+/* `iters` bfloat16 contractions back to back over n_ws weights of one shape (activations already bfloat16), timed with
+ * HIP events; the outputs stay in the handle's workspace.  epilogue: as above. */
+int candy_hip_dense_sweep(candy_hip_device *dev, const candy_hip_dense *const *ws, int n_ws, const float *dev_x,
+                          int64_t m, int epilogue, int iters, float *elapsed_ms);
+/* Layer normalization with weight and bias: (x - mean) / sqrt(mean((x - mean)^2) + eps) * w + b. */
+int candy_hip_layer_norm(candy_hip_device *dev, const float *x, const float *w, const float *b, float eps, int64_t rows,
+                         int64_t cols, float *out);
+/* x += mult * layer_norm(y) (+ step, one [cols] row added to every row; may be NULL), in place: a sublayer's result
+ * entering the residual sum through a norm of its own. */
+int candy_hip_add_layer_norm(candy_hip_device *dev, float *x, const float *y, const float *w, const float *b, float eps,
+                             float mult, const float *step, int64_t rows, int64_t cols);
+
+/* One attention layer: grouped heads, rotary positions on the first rope_dims dimensions of a head (pairs i,
+ * i + rope_dims/2; angle p * rope_base^(-2i/rope_dims)), values = the keys before rotation, scores
+ * softcap * tanh(scale * q.k / softcap), a window of positions, a per-head sink in the softmax denominator.
+ * rope_original > 0: wavelengths l = 2 pi / f longer than rope_original / rope_low use f / rope_factor, shorter than
+ * rope_original / rope_high keep f, those between are interpolated in rope_original / l. */
+typedef struct candy_hip_attn_spec {
+    int32_t n_heads, n_kv_heads, head_dim;
+    int32_t window;        /* position i attends to the last `window` positions including its own; 0: to all   */
+    int32_t rope_dims;     /* even; 0: no rotation                                                             */
+    int32_t rope_original; /* 0: no frequency scaling                                                          */
+    float scale;
+    float softcap;         /* 0: none                                                                          */
+    double rope_base, rope_factor, rope_low, rope_high;
+} candy_hip_attn_spec;
+/* Runs that layer between its projections for n tokens at positions pos0 ..: qk [n, (n_heads + n_kv_heads) * head_dim]
+ * f32 holds the projected q and k of every token; k_cache / v_cache are [n_kv_heads, max_pos, row] device arrays of the
+ * activation format, row = candy_hip_attn_row(head_dim), holding positions 0 .. pos0-1 and receiving the new ones;
+ * sink [n_heads] may be NULL; out [n, n_heads * head_dim] f32.  decode != 0 (n = 1): the kernels of the decode step. */
+int candy_hip_attn_row(int head_dim);   /* values per position and head in the cache; 0 if head_dim is unsupported */
+int candy_hip_window_attention(candy_hip_device *dev, const candy_hip_attn_spec *spec, int act, const float *qk, int64_t n,
+                               int32_t pos0, int32_t max_pos, void *k_cache, void *v_cache, const float *sink, int decode,
+                               float *out);
+
+/* ------------------------------------------------------------------ any decoder
+ * What candy_hip_llama_decode and its neighbours do, for every model of the library. */
+int candy_hip_decoder_free(candy_hip_decoder *m);
+int candy_hip_decoder_set_graph(candy_hip_decoder *m, int enable);
+int candy_hip_decoder_hidden(candy_hip_decoder *m, const float **dev_hidden);
+int candy_hip_decoder_kv_cache(candy_hip_decoder *m, void **dev_k, void **dev_v, size_t *bytes_each);
+int candy_hip_decoder_decode(candy_hip_decoder *m, int32_t token, int32_t pos, const float **dev_logits,
+                             int32_t *next_token);
+int candy_hip_decoder_decode_hidden(candy_hip_decoder *m, const float *dev_hidden, int32_t pos, const float **dev_logits,
+                                    int32_t *next_token);
+int candy_hip_decoder_generate(candy_hip_decoder *m, int32_t token, int32_t pos, int32_t n_steps, int32_t *tokens);
+int candy_hip_decoder_prefill(candy_hip_decoder *m, const int32_t *tokens, int32_t n_tokens, int32_t pos0,
+                              const float **dev_logits, int32_t *next_token);
+/* The same pass with the logits of chosen rows: rows[i] counts from the first of these tokens; dev_logits points at
+ * [n_rows, vocab], owned by the model and valid until its next call.  n_rows 0: the tokens enter the cache only. */
+int candy_hip_decoder_prefill_rows(candy_hip_decoder *m, const int32_t *tokens, int32_t n_tokens, int32_t pos0,
+                                   const int32_t *rows, int32_t n_rows, const float **dev_logits);
+/* The residual stream of every token of the last prompt pass behind the last layer, rows *row_floats apart. */
+int candy_hip_decoder_prompt_hidden(candy_hip_decoder *m, const float **dev_hidden, int64_t *row_floats);
+
+/* ------------------------------------------------------------------ Suvazen decoder
+ * x = embed[token]; every layer x += mult * norm1b(mixer(norm1(x))), then x += mult * norm2b(mlp(norm2(x))), all norms
+ * layer norms with bias; mixer: the attention above (one matrix holds the q and k rows, in that order); mlp: down .
+ * squared_relu(up . ), absent with d_ffn 0.  Layers loop_start .. loop_stop-1 run loop_times times in a row with the
+ * same weights and a cache of their own for each pass, in front of which that pass's step row is added to x.
+ * logits = logit_softcap * tanh(logit_scale * head . final_norm(x) / logit_softcap). */
+typedef struct candy_hip_suvazen candy_hip_suvazen;
+typedef struct candy_hip_suvazen_layer {
+    candy_hip_attn_spec attn;
+    int32_t d_ffn;         /* 0: no feed-forward */
+    int32_t has_sink;
+} candy_hip_suvazen_layer;
+typedef struct candy_hip_suvazen_config {
+    int32_t n_layers, d_model, vocab, max_pos;
+    int32_t loop_start, loop_stop, loop_times;   /* loop_times 0: no loop */
+    int32_t act;                                 /* enum candy_hip_act     */
+    float norm_eps, residual_mult, logit_scale, logit_softcap;
+} candy_hip_suvazen_config;
+
+enum candy_hip_suvazen_matrix {   /* bfloat16 */
+    CANDY_HIP_SV_QK = 0,     /* [(n_heads + n_kv_heads) * head_dim, d_model] */
+    CANDY_HIP_SV_O = 1,      /* [d_model, n_heads * head_dim]                */
+    CANDY_HIP_SV_UP = 2,     /* [d_ffn, d_model]                             */
+    CANDY_HIP_SV_DOWN = 3,   /* [d_model, d_ffn]                             */
+    CANDY_HIP_SV_HEAD = 4,   /* [vocab, d_model], layer = -1                 */
+    CANDY_HIP_SV_EMBED = 5   /* [vocab, d_model], layer = -1                 */
+};
+enum candy_hip_suvazen_vector {   /* f32, copied */
+    CANDY_HIP_SV_NORM1 = 0, CANDY_HIP_SV_NORM1_BIAS = 1,     /* in front of the mixer, [d_model]          */
+    CANDY_HIP_SV_NORM1B = 2, CANDY_HIP_SV_NORM1B_BIAS = 3,   /* behind it                                 */
+    CANDY_HIP_SV_NORM2 = 4, CANDY_HIP_SV_NORM2_BIAS = 5,     /* in front of the feed-forward              */
+    CANDY_HIP_SV_NORM2B = 6, CANDY_HIP_SV_NORM2B_BIAS = 7,
+    CANDY_HIP_SV_SINK = 8,                                   /* [n_heads]                                 */
+    CANDY_HIP_SV_STEP = 9,                                   /* [d_model], layer = number of the pass     */
+    CANDY_HIP_SV_FINAL = 10, CANDY_HIP_SV_FINAL_BIAS = 11    /* layer = -1                                */
+};
+int candy_hip_suvazen_create(candy_hip_device *dev, const candy_hip_suvazen_config *cfg,
+                             const candy_hip_suvazen_layer *layers, candy_hip_suvazen **out);
+candy_hip_decoder *candy_hip_suvazen_decoder(candy_hip_suvazen *m);   /* free through the decoder */
+/* Matrices are borrowed and must outlive the model. */
+int candy_hip_suvazen_set_matrix(candy_hip_suvazen *m, int which, int layer, const candy_hip_dense *w);
+int candy_hip_suvazen_set_vector(candy_hip_suvazen *m, int which, int layer, const float *host, int64_t count);
 
 /* ------------------------------------------------------------------ timing (HIP events on the handle's stream) */
 /* Runs `iters` contractions back to back, iteration i using weight ws[i % n_ws] (all the same
