@@ -339,6 +339,124 @@ def llama3_leg(dev, n_prompt=512, n_decode=128, not_eager=True):
             "tokens": toks[:8], "first_token": first_graph, "first_token_graph_equals_eager": first_graph == first_eager}
 
 
+# ------------------------------------------------------------------ --suvazen
+# Layer shapes of two common decoder sizes; both models of the leg take them.
+SUVAZEN_SIZES = {
+    "8b": dict(n_layers=32, d_model=4096, n_heads=32, n_kv_heads=8, head_dim=128, d_ffn=14336, vocab=128256),
+    "1b": dict(n_layers=16, d_model=2048, n_heads=32, n_kv_heads=8, head_dim=64, d_ffn=8192, vocab=128256),
+}
+
+
+def build_suvazen(dev, size, max_pos, window=1536, seed=600):
+    """Random-init Suvazen of a size: bfloat16 weights, one draw per shape (every layer has a device copy of its own).
+    Returns (model, bytes a decode step reads of the weights, multiply-adds per token in the layers)."""
+    from candy_amd import hip, suvazen
+    c = size
+    mixer = {"heads": c["n_heads"], "kv_heads": c["n_kv_heads"], "dim": c["head_dim"], "scale": c["head_dim"] ** -0.5,
+             "softcap": 40.0, "mask": {"size": window},
+             "rot": {"base": 500000.0, "dims": c["head_dim"] // 2,
+                     "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}
+    cfg = {"vocab": c["vocab"], "width": c["d_model"], "norm": {"eps": 1e-5}, "residual_mult": 0.5, "logit_scale": 1.0,
+           "logit_softcap": 25.0, "layers": [{"type": "attention", "mixer": mixer, "mlp": {"kind": "dense", "ff": c["d_ffn"]}}
+                                             for _ in range(c["n_layers"])]}
+    rng = np.random.Generator(np.random.Philox(seed))
+    draws = {}
+
+    class Tensors:
+        def __contains__(self, name):
+            return True
+
+        def bits(self, name):
+            kind = name.rsplit(".", 1)[-1]
+            qd, kd, d, ff = c["n_heads"] * c["head_dim"], c["n_kv_heads"] * c["head_dim"], c["d_model"], c["d_ffn"]
+            shape = {"q": (qd, d), "k": (kd, d), "o": (d, qd), "up": (ff, d), "down": (d, ff), "embed": (c["vocab"], d),
+                     "head": (c["vocab"], d)}[kind]
+            if kind not in draws:
+                draws[kind] = hip.bf16_bits(rng.standard_normal(shape, dtype=np.float32) * np.float32(0.02))
+            return draws[kind]
+
+        def f32(self, name):
+            if name.endswith("sink"):
+                return np.zeros(c["n_heads"], np.float32)
+            return np.zeros(c["d_model"], np.float32) if name.endswith(".b") else np.ones(c["d_model"], np.float32)
+
+    model = suvazen.build(dev, cfg, Tensors(), max_pos)
+    qk = (c["n_heads"] + c["n_kv_heads"]) * c["head_dim"]
+    layer = c["d_model"] * (qk + c["n_heads"] * c["head_dim"] + 2 * c["d_ffn"])
+    return model, 2 * (layer * c["n_layers"] + c["vocab"] * c["d_model"]), layer * c["n_layers"]
+
+
+def build_llama_like(dev, size, max_pos, seed=8100):
+    """The Llama decoder of the same size (Q4_K, Q6_K down and head, Q8_0 embedding rows), random blocks."""
+    from candy_amd import hip, synth
+    c = size
+    model = hip.Llama(dev, **c, max_pos=max_pos, rms_eps=1e-5, rope_base=500000.0)
+    qd, kd, d, ff = c["n_heads"] * c["head_dim"], c["n_kv_heads"] * c["head_dim"], c["d_model"], c["d_ffn"]
+    shapes = [(hip.W_Q, qd, d, synth.Q4_K), (hip.W_K, kd, d, synth.Q4_K), (hip.W_V, kd, d, synth.Q4_K), (hip.W_O, d, qd, synth.Q4_K),
+              (hip.W_GATE, ff, d, synth.Q4_K), (hip.W_UP, ff, d, synth.Q4_K), (hip.W_DOWN, d, ff, synth.Q6_K)]
+    draws, nbytes = {}, 0
+    for l in range(c["n_layers"]):
+        for kind, r, k, f in shapes:
+            if kind not in draws:
+                draws[kind] = synth.random_weight(f, r, k, seed + kind, synth.unit_scale(f))
+            model.set_qweight(kind, l, dev.qtensor(f, r, k, draws[kind]))
+            nbytes += synth.weight_nbytes(f, r, k)
+        for kind in (hip.W_ATTN_NORM, hip.W_FFN_NORM):
+            model.set_norm(kind, l, np.ones(d, np.float32))
+    model.set_norm(hip.W_OUT_NORM, -1, np.ones(d, np.float32))
+    for kind, f in ((hip.W_HEAD, synth.Q6_K), (hip.W_EMBED, synth.Q8_0)):
+        model.set_qweight(kind, -1, dev.qtensor(f, c["vocab"], d, synth.random_weight(f, c["vocab"], d, seed + kind, synth.unit_scale(f))))
+    macs = c["n_layers"] * d * (2 * qd + 2 * kd + 3 * ff)
+    return model, nbytes + synth.weight_nbytes(synth.Q6_K, c["vocab"], d), macs
+
+
+def suvazen_leg(dev, sizes, prompts=(512, 2048), n_decode=64, models=("suvazen", "llama"), eager=False):
+    """Prefill and decode of the Suvazen decoder beside the Llama decoder at equal layer shapes."""
+    out = {}
+    for name in sizes:
+        size, res = SUVAZEN_SIZES[name], {}
+        window = 1536
+        for which in models:
+            log(f"building {which} {name} ...")
+            max_pos = max(prompts) + n_decode + 8
+            if which == "suvazen":
+                model, wbytes, macs = build_suvazen(dev, size, max_pos, window)
+            else:
+                model, wbytes, macs = build_llama_like(dev, size, max_pos)
+            if eager:
+                model.set_graph(False)
+            rows = []
+            for n in prompts:
+                prompt = [int(t) for t in np.random.default_rng(n).integers(0, size["vocab"], n)]
+                for _ in range(6):
+                    tok, _ = model.prefill(prompt, 0, want_logits=False)
+                dev.synchronize()
+                reps = 5
+                t0 = time.perf_counter()
+                for _ in range(reps):
+                    tok, _ = model.prefill(prompt, 0, want_logits=False)
+                dev.synchronize()
+                pre = (time.perf_counter() - t0) / reps
+                model.generate(tok, n, 4)
+                t0 = time.perf_counter()
+                model.generate(tok, n, n_decode)
+                dev.synchronize()
+                dec = (time.perf_counter() - t0) / n_decode
+                # the Llama decoder's cache is f32, Suvazen's bfloat16 and read within the window only
+                seen = n + n_decode // 2
+                kv = 2 * size["n_layers"] * size["n_kv_heads"] * size["head_dim"] * (min(seen, window) * 2 if which == "suvazen" else seen * 4)
+                bpt = wbytes + kv
+                rows.append({"prompt": n, "prefill_ms": round(pre * 1e3, 3), "prefill_tok_s": round(n / pre, 1),
+                             "prefill_linear_TFLOPs": round(2.0 * macs * n / pre / 1e12, 1),
+                             "decode_ms_per_token": round(dec * 1e3, 4), "decode_tok_s": round(1 / dec, 2),
+                             "decode_bytes_per_token": bpt, "decode_hbm_frac": round(bpt / dec / 1e9 / HBM_PEAK_GBPS, 4)})
+                log(f"  {which} {name}: {rows[-1]}")
+            res[which] = rows
+            model.free()
+        out[name] = res
+    return out
+
+
 def prefill_kv(dev, model, cfg, n_pos, seed=9):
     """KV cache positions [0, n_pos) <- N(0,1), in the cache's element type (f32, or fp16 after set_kv_f16)."""
     from candy_amd import hip
@@ -420,6 +538,10 @@ def main():
                     help="untimed calls in front of them, as milliseconds of work (the matrix-core kernels run 10-20 %% "
                          "slower until the chip has raised its clocks); a counter run wants few dispatches: 0")
     ap.add_argument("--no-llama3", action="store_true", help="skip the Llama-3-8B-shaped prefill + decode leg")
+    ap.add_argument("--suvazen", nargs="?", const="8b,1b", metavar="SIZES",
+                    help="instead of the default workload: prefill and decode of the Suvazen decoder beside the Llama decoder at "
+                         "equal layer shapes (sizes: 8b, 1b)")
+    ap.add_argument("--suvazen-models", default="suvazen,llama", help="which decoders --suvazen runs")
     ap.add_argument("--decode-steps", type=int, default=32)
     ap.add_argument("--eager", action="store_true",
                     help="decoders launch their kernels one by one instead of replaying a captured HIP graph (for "
@@ -446,6 +568,11 @@ def main():
         dev.set_option(key, int(val))
     if args.eager:
         dev.set_option("llama.graph", 0)
+    if args.suvazen:
+        legs = suvazen_leg(dev, args.suvazen.split(","), models=args.suvazen_models.split(","), eager=args.eager)
+        dev.close()
+        print(json.dumps({"metric": "Suvazen prefill and decode beside Llama", "data": "synthetic", "n_gpus": 1, "legs": legs}))
+        return
     fmt, rows, cols = synth.Q4_K, 4096, 11008
     alg = algorithmic_bytes(fmt, rows, cols)
     if args.calibrate_copy:

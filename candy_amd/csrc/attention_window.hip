@@ -79,6 +79,46 @@ __global__ __launch_bounds__(256) void k_rope_cache(const RopeArgs a, AT *__rest
     }
 }
 
+// The same for heads whose halves are multiples of four values: one thread per four pairs, or four values that pass.
+template <class AT>
+__global__ __launch_bounds__(256) void k_rope_cache4(const RopeArgs a, AT *__restrict__ q, AT *__restrict__ kc, AT *__restrict__ vc,
+                                                     int n, int pos0) {
+    typedef AT at4 __attribute__((ext_vector_type(4)));
+    const int slots = a.H + a.G, pairs = a.half >> 2, items = pairs + ((a.row - 2 * a.half) >> 2);
+    const int64_t idx = (int64_t)blockIdx.x * 256 + threadIdx.x;
+    if (idx >= (int64_t)n * slots * items) return;
+    const int item = (int)(idx % items);
+    const int slot = (int)(idx / items % slots);
+    const int t = (int)(idx / ((int64_t)items * slots));
+    const int pos = pos0 + t;
+    const float *head = a.qk + (size_t)t * a.qk_ld + (size_t)slot * a.dim;
+    auto load = [&](int i) {
+        f32x4 v = *(const f32x4 *)(head + i);
+        for (int c = 1; c < a.qk_copies; ++c) v += *(const f32x4 *)(head + (size_t)c * a.qk_stride + i);
+        return v;
+    };
+    const bool is_q = slot < a.H;
+    const size_t cache = (size_t)(slot - a.H) * a.kv_stride + (size_t)pos * a.row;
+    AT *dst = is_q ? q + ((size_t)t * a.H + slot) * a.row : kc + cache;
+    if (item < pairs) {
+        const int i = item * 4;
+        const f32x4 u = load(i), v = load(i + a.half);
+        const f32x4 c = *(const f32x4 *)(a.cos_t + (size_t)pos * a.half + i), s = *(const f32x4 *)(a.sin_t + (size_t)pos * a.half + i);
+        *(at4 *)(dst + i) = __builtin_convertvector(u * c - v * s, at4);
+        *(at4 *)(dst + i + a.half) = __builtin_convertvector(v * c + u * s, at4);
+        if (!is_q) {
+            *(at4 *)(vc + cache + i) = __builtin_convertvector(u, at4);
+            *(at4 *)(vc + cache + i + a.half) = __builtin_convertvector(v, at4);
+        }
+    } else {
+        const int i = 2 * a.half + (item - pairs) * 4;
+        const f32x4 u = i < a.dim ? load(i) : f32x4{0.f, 0.f, 0.f, 0.f};
+        const at4 o = __builtin_convertvector(u, at4);
+        *(at4 *)(dst + i) = o;
+        if (!is_q) *(at4 *)(vc + cache + i) = o;
+    }
+}
+
 struct WindowArgs {
     const float *sink;
     int H, G, dim, row, window, out_cols;
@@ -299,6 +339,17 @@ __global__ __launch_bounds__(256, 2) void k_window_attn_prompt(const WindowArgs 
 // wavefront attends to them from LDS.
 constexpr int DEC_UNR = 4;
 
+// Sum over groups of LPR neighbouring lanes, in every lane of the group, on the DPP path.
+template <int LPR>
+__device__ __forceinline__ float lanes_sum(float v) {
+    v += dpp_move<0xB1>(v);                       // quad_perm [1,0,3,2]
+    v += dpp_move<0x4E>(v);                       // quad_perm [2,3,0,1]
+    if (LPR >= 8) v += dpp_move<0x141>(v);        // row_half_mirror
+    if (LPR >= 16) v += dpp_move<0x140>(v);       // row_mirror
+    if (LPR >= 32) v += __shfl_xor(v, 16, 64);
+    return v;
+}
+
 template <int LPR> constexpr int dec_batch() { return 4 * (64 / LPR) * DEC_UNR; }
 
 template <int LPR, int GROUP>
@@ -306,7 +357,7 @@ __global__ __launch_bounds__(256) void k_window_attn_decode(const WindowArgs a, 
                                                             const int *__restrict__ pos_ptr, float *__restrict__ part, int n_splits) {
     constexpr int RPW = 64 / LPR, BATCH = dec_batch<LPR>(), W = LPR * 8, SLOTS = 4 * RPW;
     __shared__ __align__(16) float sq[GROUP + 2][W];   // rotated queries, then the new token's key and value
-    __shared__ float sm[SLOTS][GROUP], sl[SLOTS][GROUP];
+    __shared__ float sm[SLOTS][GROUP], sl[SLOTS][GROUP], tot[GROUP][2];
     __shared__ __align__(16) float so[SLOTS][GROUP][W];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int kvh = blockIdx.x, split = blockIdx.y, ratio = a.H / a.G, h0 = blockIdx.z * GROUP;
@@ -314,9 +365,32 @@ __global__ __launch_bounds__(256) void k_window_attn_decode(const WindowArgs a, 
     const bool chunk = cl * 8 < a.row;                // rows narrower than LPR chunks leave lanes idle
     const int coff = chunk ? cl * 8 : 0;
     bf16 *kh = kc + (size_t)kvh * a.kv_stride, *vh = vc + (size_t)kvh * a.kv_stride;
+    const bool fresh = split == 0;
+    // Requested in the order they become possible: the projected rows at once, what depends on the position behind it,
+    // the cache rows last, so that the rotation below does not wait for them.
+    constexpr int PER = ((GROUP + 2) * W + 255) / 256;
+    const int rows = GROUP + (fresh ? 2 : 0);
+    float plain[PER], other[PER];
+#pragma unroll
+    for (int j = 0; j < PER; ++j) {
+        const int i = tid + 256 * j, r = i / W, c = i % W;
+        const bool used = r < rows && c < a.dim;
+        const float *head = ra.qk + (size_t)(r < GROUP ? kvh * ratio + min(h0 + r, ratio - 1) : a.H + kvh) * a.dim;
+        plain[j] = used ? head[c] : 0.0f;
+        other[j] = used && c < 2 * ra.half ? head[c < ra.half ? c + ra.half : c - ra.half] : 0.0f;
+    }
     const int pos = *pos_ptr;
     const int lo = max(0, pos - a.window + 1);        // positions lo .. pos-1 are in the cache
     const int cached = pos - lo;
+    float cs[PER], sn[PER];
+#pragma unroll
+    for (int j = 0; j < PER; ++j) {
+        const int i = tid + 256 * j, r = i / W, c = i % W;
+        const bool used = r <= GROUP && r < rows && c < 2 * ra.half;
+        const size_t at = (size_t)pos * ra.half + (c < ra.half ? c : c - ra.half);
+        cs[j] = used ? ra.cos_t[at] : 1.0f;
+        sn[j] = used ? ra.sin_t[at] : 0.0f;
+    }
     u32x4v kv[DEC_UNR], vv[DEC_UNR];
     auto fetch = [&](int b) __attribute__((always_inline)) {
 #pragma unroll
@@ -327,16 +401,13 @@ __global__ __launch_bounds__(256) void k_window_attn_decode(const WindowArgs a, 
             vv[u] = __builtin_nontemporal_load((const u32x4v *)(vh + off));
         }
     };
-    fetch(split);  // in flight while the queries are rotated
-    const bool fresh = split == 0;
-    for (int i = tid; i < (GROUP + (fresh ? 2 : 0)) * W; i += 256) {
-        const int r = i / W, c = i % W;
-        float v = 0.0f;
-        if (c < a.dim) {
-            const int slot = r < GROUP ? kvh * ratio + min(h0 + r, ratio - 1) : a.H + kvh;
-            v = qk_at(ra, ra.qk, slot, c);
-            if (r <= GROUP) v = rotated(ra, ra.qk, slot, c, pos, v);
-        }
+    fetch(split);
+    __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+    for (int j = 0; j < PER; ++j) {
+        const int i = tid + 256 * j, r = i / W, c = i % W;
+        if (r >= rows) continue;
+        float v = c < ra.half ? plain[j] * cs[j] - other[j] * sn[j] : plain[j] * cs[j] + other[j] * sn[j];
         if (r >= GROUP) {
             const bf16 b = (bf16)v;  // attend to the rows as the cache holds them
             v = (float)b;
@@ -345,6 +416,7 @@ __global__ __launch_bounds__(256) void k_window_attn_decode(const WindowArgs a, 
         sq[r][c] = v;
     }
     __syncthreads();
+    const float c_in = a.cap > 0.0f ? a.scale / a.cap : a.scale * LOG2E, c_out = a.cap * LOG2E;
     float qf[GROUP][8], m[GROUP], l[GROUP], o[GROUP][8];
 #pragma unroll
     for (int q = 0; q < GROUP; ++q) {
@@ -352,7 +424,7 @@ __global__ __launch_bounds__(256) void k_window_attn_decode(const WindowArgs a, 
         l[q] = 0.0f;
 #pragma unroll
         for (int e = 0; e < 8; ++e) {
-            qf[q][e] = chunk ? sq[q][cl * 8 + e] * a.scale : 0.0f;
+            qf[q][e] = chunk ? sq[q][cl * 8 + e] * c_in : 0.0f;
             o[q][e] = 0.0f;
         }
     }
@@ -360,10 +432,8 @@ __global__ __launch_bounds__(256) void k_window_attn_decode(const WindowArgs a, 
         float d = 0.0f;
 #pragma unroll
         for (int e = 0; e < 8; ++e) d = fmaf(qf[q][e], k[e], d);
-#pragma unroll
-        for (int x = 1; x < LPR; x <<= 1) d += __shfl_xor(d, x, 64);
-        if (a.cap > 0.0f) d = a.cap * tanh_fast(d / a.cap);
-        return d * LOG2E;
+        d = lanes_sum<LPR>(d);
+        return a.cap > 0.0f ? c_out * tanh_fast(d) : d;
     };
     for (int b = split; b * BATCH < cached; b += n_splits) {
         float kf[DEC_UNR][8], vf[DEC_UNR][8];
@@ -434,23 +504,30 @@ __global__ __launch_bounds__(256) void k_window_attn_decode(const WindowArgs a, 
         for (int e = 0; e < 8; ++e) so[slot][q][cl * 8 + e] = o[q][e];
     }
     __syncthreads();
+    // a wavefront's lanes hold one slot each: the factor of every slot, once
+    for (int q = wave; q < GROUP; q += 4) {
+        const float ms = lane < SLOTS ? sm[lane][q] : LOW;
+        const float mm = wave_max(ms), f = __builtin_amdgcn_exp2f(ms - mm);
+        const float ll = wave_sum(lane < SLOTS ? sl[lane][q] * f : 0.0f);
+        if (lane < SLOTS) sm[lane][q] = f;
+        if (lane == 0) {
+            tot[q][0] = mm;
+            tot[q][1] = ll;
+        }
+    }
+    __syncthreads();
     for (int i = tid; i < GROUP * W; i += 256) {
         const int q = i / W, c = i % W;
         if (h0 + q >= ratio || c >= a.row) continue;
-        float mm = LOW;
-        for (int s = 0; s < SLOTS; ++s) mm = fmaxf(mm, sm[s][q]);
-        float ll = 0.0f, oo = 0.0f;
-        for (int s = 0; s < SLOTS; ++s) {
-            const float f = __builtin_amdgcn_exp2f(sm[s][q] - mm);
-            ll += sl[s][q] * f;
-            oo += so[s][q][c] * f;
-        }
+        float oo = 0.0f;
+#pragma unroll
+        for (int s = 0; s < SLOTS; ++s) oo += so[s][q][c] * sm[s][q];
         // per (head, split): row values, then the maximum and the sum
-        float *p = part + ((size_t)(kvh * ratio + h0 + q) * n_splits + split) * (a.row + 2);
+        float *p = part + ((size_t)(kvh * ratio + h0 + q) * n_splits + split) * (a.row + 4);
         p[c] = oo;
         if (c == 0) {
-            p[a.row] = mm;
-            p[a.row + 1] = ll;
+            p[a.row] = tot[q][0];
+            p[a.row + 1] = tot[q][1];
         }
     }
 }
@@ -458,24 +535,45 @@ __global__ __launch_bounds__(256) void k_window_attn_decode(const WindowArgs a, 
 // one workgroup per head; at most 64 splits, a lane each for the maxima
 __global__ __launch_bounds__(256) void k_window_attn_merge(const WindowArgs a, const float *__restrict__ part, int n_splits,
                                                            bf16 *__restrict__ out) {
-    __shared__ float f[64];
+    constexpr int MAX_SPLITS = 64;
+    __shared__ __align__(16) f32x4 red[256];
     const int h = blockIdx.x, tid = threadIdx.x, lane = tid & 63;
-    const float *p = part + (size_t)h * n_splits * (a.row + 2);
+    // the head's partial outputs as 16-byte loads: thread (sg, c4) takes columns 4 c4 .. of splits sg, sg + SG, ...
+    const int pitch = a.row + 4, C4 = a.row >> 2, SG = 256 / C4, c4 = tid % C4, sg = tid / C4;
+    const float *p = part + (size_t)h * n_splits * pitch;
     float ms = LOW, ls = 0.0f;
     if (lane < n_splits) {
-        ms = p[(size_t)lane * (a.row + 2) + a.row];
-        ls = p[(size_t)lane * (a.row + 2) + a.row + 1];
+        ms = p[(size_t)lane * pitch + a.row];
+        ls = p[(size_t)lane * pitch + a.row + 1];
     }
     const float sink = a.sink ? a.sink[h] * LOG2E : MASKED;
+    constexpr int AHEAD = 8;
+    f32x4 v[AHEAD];
+#pragma unroll
+    for (int j = 0; j < AHEAD; ++j) v[j] = *(const f32x4 *)(p + (size_t)min(sg + SG * j, n_splits - 1) * pitch + 4 * c4);
+    __builtin_amdgcn_sched_barrier(0);  // every load above is requested before anything below waits
     const float m = fmaxf(wave_max(ms), sink);
     const float w = lane < n_splits ? __builtin_amdgcn_exp2f(ms - m) : 0.0f;
     const float l = wave_sum(ls * w) + (a.sink ? __builtin_amdgcn_exp2f(sink - m) : 0.0f);
-    if (tid < 64) f[lane] = w / l;
+    const float f = w / l;
+    f32x4 o{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int j = 0; j < AHEAD; ++j) {
+        const int s = sg + SG * j;
+        const float fs = __shfl(f, min(s, 63), 64);
+        o += v[j] * (s < n_splits ? fs : 0.0f);
+    }
+    for (int j = AHEAD; SG * j < MAX_SPLITS; ++j) {
+        const int s = sg + SG * j;
+        const float fs = __shfl(f, min(s, 63), 64);
+        if (s < n_splits) o += *(const f32x4 *)(p + (size_t)s * pitch + 4 * c4) * fs;
+    }
+    red[tid] = o;
     __syncthreads();
     for (int c = tid; c < a.dim; c += 256) {
-        float o = 0.0f;
-        for (int s = 0; s < n_splits; ++s) o += p[(size_t)s * (a.row + 2) + c] * f[s];
-        out[(size_t)h * a.dim + c] = (bf16)o;
+        float t = 0.0f;
+        for (int g = 0; g < SG; ++g) t += red[g * C4 + (c >> 2)][c & 3];
+        out[(size_t)h * a.dim + c] = (bf16)t;
     }
     if (h == a.H - 1)
         for (int i = a.H * a.dim + tid; i < a.out_cols; i += 256) out[i] = (bf16)0.0f;
@@ -535,7 +633,7 @@ int window_splits(const candy_hip_device *dev, const candy_hip_attn_spec &s, int
 }
 
 size_t window_scratch_floats(const candy_hip_attn_spec &s, int n_splits) {
-    return (size_t)s.n_heads * n_splits * (attn_row(s.head_dim) + 2);
+    return (size_t)s.n_heads * n_splits * (attn_row(s.head_dim) + 4);
 }
 
 static WindowArgs window_args(const WindowAttn &A) {
@@ -560,9 +658,22 @@ static RopeArgs rope_args(const WindowAttn &A) {
 }
 
 static int launch_rope(candy_hip_device *dev, const WindowAttn &A, int n, int pos0, const int *pos_ptr) {
+    const RopeArgs ra = rope_args(A);
+    if (!pos_ptr && A.s.head_dim % 4 == 0 && ra.half % 4 == 0 && ra.qk_ld % 4 == 0 && ((uintptr_t)ra.qk & 15) == 0 && ra.qk_stride % 4 == 0) {
+        const int64_t items = (ra.half >> 2) + ((A.row - 2 * ra.half) >> 2);
+        const int64_t grid = ((int64_t)n * (ra.H + ra.G) * items + 255) / 256;
+        CANDY_REQUIRE(grid <= 0x7FFFFFFF, "prompt too long for one pass");
+        if (A.f32)
+            hipLaunchKernelGGL((k_rope_cache4<float>), dim3((unsigned)grid), dim3(256), 0, dev->stream, ra, (float *)A.q,
+                               (float *)A.k_cache, (float *)A.v_cache, n, pos0);
+        else
+            hipLaunchKernelGGL((k_rope_cache4<bf16>), dim3((unsigned)grid), dim3(256), 0, dev->stream, ra, (bf16 *)A.q,
+                               (bf16 *)A.k_cache, (bf16 *)A.v_cache, n, pos0);
+        CANDY_LAUNCH_CHECK();
+        return CANDY_HIP_OK;
+    }
     const int64_t grid = ((int64_t)n * (A.s.n_heads + A.s.n_kv_heads) * A.row + 255) / 256;
     CANDY_REQUIRE(grid <= 0x7FFFFFFF, "prompt too long for one pass");
-    const RopeArgs ra = rope_args(A);
     if (A.f32)
         hipLaunchKernelGGL((k_rope_cache<float>), dim3((unsigned)grid), dim3(256), 0, dev->stream, ra, (float *)A.q,
                            (float *)A.k_cache, (float *)A.v_cache, n, pos0, pos_ptr);
@@ -620,7 +731,7 @@ int launch_window_decode(candy_hip_device *dev, const WindowAttn &A, const int *
         if (int rc = launch_rope(dev, A, 1, 0, pos_ptr)) return rc;
         return launch_rows(dev, A, 1, 0, pos_ptr);
     }
-    CANDY_REQUIRE(A.n_splits >= 1 && A.n_splits <= 64, "internal: attention splits");
+    CANDY_REQUIRE(A.n_splits >= 1 && A.n_splits <= 64 && A.qk.copies == 1, "internal: attention launch");
     const int group = group_of(A.s);
     switch (lanes_per_row(A.row)) {
     case 4: launch_dec<4>(dev, A, group, pos_ptr); break;

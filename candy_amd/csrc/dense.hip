@@ -47,30 +47,53 @@ __device__ __forceinline__ void lds8(const float *p, float (&f)[8]) {
 }
 
 // ------------------------------------------------------------------ one row
-constexpr int MV_STEP = 2048;  // K values a wavefront takes per step: 4 x 64 lanes x 8
+// The norms in front of the contraction (launch_norm_chain's arithmetic), for a kernel that runs them in its prologue.
+struct NormPro {
+    const float *x, *y, *post_w, *post_b, *step, *pre_w, *pre_b;
+    float *x_out;
+    float mult, eps;
+    int cols;
+};
+
+__device__ __forceinline__ float pro_sum(float v, float *red) {
+    v = wave_sum(v);
+    __syncthreads();  // the last use of red is over
+    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
+    __syncthreads();
+    const int n = blockDim.x >> 6;
+    float t = red[0];
+    for (int w = 1; w < n; ++w) t += red[w];
+    return t;
+}
 
 template <class AT> constexpr int mv_lds_values() { return sizeof(AT) == 2 ? 16384 : 8192; }  // 32 KB: whole steps
+template <int R> constexpr int mv_unroll() { return 8 / R; }                                  // 8 KB requested per step
 
-// R rows per wavefront; the next step's weights are requested before the current ones are multiplied, the first ones
-// before the activations are staged.
-template <class AT, int R, int EPI>
-__global__ __launch_bounds__(512) void k_dense_mv(const AT *__restrict__ x, const bf16 *__restrict__ W, void *__restrict__ yv,
-                                                  int K, int n_store, const EpiArgs ea) {
-    constexpr int U = 4, CH = mv_lds_values<AT>();
+// One workgroup of W wavefronts per CU where the rows go round (launch_mv picks W and R so that they do), R weight rows
+// per wavefront.  The next step's weights are requested before the current ones are multiplied, the first ones before
+// the activations are staged.  NV > 0: the activations are made here, by the norm chain in front of the contraction
+// (NV float4 per thread); every workgroup repeats it, workgroup 0 writes the new residual row.
+template <class AT, int R, int EPI, int NV>
+__global__ __launch_bounds__(1024) void k_dense_mv(const AT *__restrict__ x, const bf16 *__restrict__ W, void *__restrict__ yv,
+                                                   int K, int rows, int n_store, const EpiArgs ea, const NormPro np) {
+    constexpr int U = mv_unroll<R>(), STEP = U * 512, CH = mv_lds_values<AT>();
     __shared__ __align__(16) AT xs[CH];
-    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-    const int row0 = (blockIdx.x * 8 + wave) * R;
-    const bf16 *wr = W + (size_t)row0 * K + lane * 8;
-    const int last = K - 8 - lane * 8;  // largest step offset this lane may load at
+    __shared__ float red[16];
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int threads = blockDim.x;
+    const int row0 = (blockIdx.x * (threads >> 6) + wave) * R;
     float acc[R];
 #pragma unroll
     for (int r = 0; r < R; ++r) acc[r] = 0.0f;
+    const bf16 *wr[R];
+#pragma unroll
+    for (int r = 0; r < R; ++r) wr[r] = W + (size_t)min(row0 + r, rows - 1) * K;
     auto fetch = [&](u32x4v (&w)[R][U], int k0) __attribute__((always_inline)) {
 #pragma unroll
         for (int u = 0; u < U; ++u) {
-            const int k = max(min(k0 + u * 512, last), -lane * 8);  // past the row: any value of it, times x = 0
+            const int k = min(k0 + u * 512 + lane * 8, K - 8);  // past the row: any value of it, times x = 0
 #pragma unroll
-            for (int r = 0; r < R; ++r) w[r][u] = __builtin_nontemporal_load((const u32x4v *)(wr + (size_t)r * K + k));
+            for (int r = 0; r < R; ++r) w[r][u] = __builtin_nontemporal_load((const u32x4v *)(wr[r] + k));
         }
     };
     auto multiply = [&](const u32x4v (&w)[R][U], int k0) __attribute__((always_inline)) {
@@ -90,21 +113,83 @@ __global__ __launch_bounds__(512) void k_dense_mv(const AT *__restrict__ x, cons
     };
     auto stage = [&](int k0) __attribute__((always_inline)) {
         if (k0) __syncthreads();  // the previous chunk is consumed
-        const int n = min(CH, (K - k0 + MV_STEP - 1) / MV_STEP * MV_STEP);
+        const int n = min(CH, (K - k0 + STEP - 1) / STEP * STEP);
         constexpr int PER = 16 / sizeof(AT);
-        for (int i = tid * PER; i < n; i += 512 * PER)
+        for (int i = tid * PER; i < n; i += threads * PER)
             *(u32x4v *)&xs[i] = k0 + i < K ? *(const u32x4v *)(x + k0 + i) : u32x4v{0, 0, 0, 0};
         __syncthreads();
     };
     u32x4v wa[R][U], wb[R][U];
-    fetch(wa, 0);
-    for (int k0 = 0; k0 < K; k0 += 2 * MV_STEP) {
-        if ((k0 & (CH - 1)) == 0) stage(k0);
-        if (k0 + MV_STEP < K) fetch(wb, k0 + MV_STEP);
+    if constexpr (NV > 0) {
+        f32x4 xv[NV], yv4[NV];
+        const f32x4 zero{0.f, 0.f, 0.f, 0.f};
+        auto load = [&](const float *p, f32x4 (&d)[NV]) __attribute__((always_inline)) {
+#pragma unroll
+            for (int i = 0; i < NV; ++i) d[i] = (tid + threads * i) * 4 < K ? *(const f32x4 *)(p + (tid + threads * i) * 4) : zero;
+        };
+        f32x4 wv[NV], bv[NV], pw[NV], pb[NV];
+        load(np.x, xv);
+        if (np.y) {
+            load(np.y, yv4);
+            load(np.post_w, pw);
+            load(np.post_b, pb);
+        }
+        load(np.pre_w, wv);
+        load(np.pre_b, bv);
+        fetch(wa, 0);
+        const float inv_n = 1.0f / (float)np.cols;
+        auto normalize = [&](f32x4 (&d)[NV], const f32x4 (&w)[NV], const f32x4 (&b)[NV]) __attribute__((always_inline)) {
+            float s = 0.0f;
+#pragma unroll
+            for (int i = 0; i < NV; ++i) s += (d[i][0] + d[i][1]) + (d[i][2] + d[i][3]);
+            const float mean = pro_sum(s, red) * inv_n;
+            float q = 0.0f;
+#pragma unroll
+            for (int i = 0; i < NV; ++i)
+#pragma unroll
+                for (int j = 0; j < 4; ++j) {
+                    d[i][j] = (tid + threads * i) * 4 + j < np.cols ? d[i][j] - mean : 0.0f;
+                    q += d[i][j] * d[i][j];
+                }
+            const float rstd = 1.0f / sqrtf(pro_sum(q, red) * inv_n + np.eps);
+#pragma unroll
+            for (int i = 0; i < NV; ++i)
+#pragma unroll
+                for (int j = 0; j < 4; ++j) d[i][j] = d[i][j] * rstd * w[i][j] + b[i][j];  // w = b = 0 past the row
+        };
+        if (np.y) {
+            normalize(yv4, pw, pb);
+#pragma unroll
+            for (int i = 0; i < NV; ++i) xv[i] += np.mult * yv4[i];
+        }
+        if (np.step) {
+            load(np.step, yv4);
+#pragma unroll
+            for (int i = 0; i < NV; ++i) xv[i] += yv4[i];
+        }
+        if (np.x_out && blockIdx.x == 0) {
+#pragma unroll
+            for (int i = 0; i < NV; ++i)
+                if ((tid + threads * i) * 4 < K) *(f32x4 *)(np.x_out + (tid + threads * i) * 4) = xv[i];
+        }
+        normalize(xv, wv, bv);
+        typedef AT at4 __attribute__((ext_vector_type(4)));
+        const int n = (K + STEP - 1) / STEP * STEP;
+#pragma unroll
+        for (int i = 0; i < NV; ++i)
+            if ((tid + threads * i) * 4 < n) *(at4 *)&xs[(tid + threads * i) * 4] = __builtin_convertvector(xv[i], at4);
+        for (int i = (tid + threads * NV) * 4; i < n; i += threads * 4) *(at4 *)&xs[i] = __builtin_convertvector(zero, at4);
+        __syncthreads();
+    } else {
+        fetch(wa, 0);
+    }
+    for (int k0 = 0; k0 < K; k0 += 2 * STEP) {
+        if (NV == 0 && (k0 & (CH - 1)) == 0) stage(k0);
+        if (k0 + STEP < K) fetch(wb, k0 + STEP);
         multiply(wa, k0);
-        if (k0 + MV_STEP >= K) break;
-        if (k0 + 2 * MV_STEP < K) fetch(wa, k0 + 2 * MV_STEP);
-        multiply(wb, k0 + MV_STEP);
+        if (k0 + STEP >= K) break;
+        if (k0 + 2 * STEP < K) fetch(wa, k0 + 2 * STEP);
+        multiply(wb, k0 + STEP);
     }
     float mine = 0.0f;
 #pragma unroll
@@ -273,29 +358,77 @@ __global__ __launch_bounds__(256) void k_dense_mm_f32(const bf16 *__restrict__ W
 }
 
 // ------------------------------------------------------------------ launches
-template <class AT, int R>
-static void launch_mv_epi(candy_hip_device *dev, const DenseLaunch &L) {
-    const dim3 g((unsigned)(L.w->rows_pad / (8 * R))), b(512);
+struct MvShape {
+    int waves, rows;  // wavefronts per workgroup, weight rows per wavefront
+};
+
+// Rows over wavefronts: with up to 64 rows per CU one workgroup per CU takes them all, its shape the one that leaves the
+// fewest slots empty (the more wavefronts the better, from eight on); longer weights take many workgroups of 8 x 4.
+static MvShape mv_shape(const candy_hip_device *dev, int64_t rows) {
+    const int64_t per_cu = (rows + dev->num_cus - 1) / dev->num_cus;
+    if (per_cu > 64) return {8, 4};
+    if (per_cu <= 8) return {8, 1};
+    MvShape best{16, 4};
+    int64_t best_cost = 1 << 30;
+    for (int r : {1, 2, 4})
+        for (int w = 8; w <= 16; ++w) {
+            const int64_t slots = (int64_t)w * r;
+            if (slots < per_cu) continue;
+            const int64_t cost = (slots - per_cu) * 64 - w;
+            if (cost < best_cost) { best_cost = cost; best = {w, r}; }
+        }
+    return best;
+}
+
+template <class AT, int R, int EPI>
+static void launch_mv_nv(candy_hip_device *dev, const DenseLaunch &L, int waves, int nv, const NormPro &np) {
+    const int64_t per_wg = (int64_t)waves * R;
+    const dim3 g((unsigned)((L.n_store + per_wg - 1) / per_wg)), b((unsigned)(64 * waves));
     const EpiArgs ea{L.scale, L.cap};
     const AT *x = (const AT *)L.x;
     const bf16 *W = (const bf16 *)L.w->data;
-    const int K = (int)L.w->ld, ns = (int)L.n_store;
+    const int K = (int)L.w->ld, rows = (int)L.w->rows_pad, ns = (int)L.n_store;
+    if constexpr (sizeof(AT) == 2) {
+        switch (nv) {
+        case 1: hipLaunchKernelGGL((k_dense_mv<AT, R, EPI, 1>), g, b, 0, dev->stream, x, W, L.y, K, rows, ns, ea, np); return;
+        case 2: hipLaunchKernelGGL((k_dense_mv<AT, R, EPI, 2>), g, b, 0, dev->stream, x, W, L.y, K, rows, ns, ea, np); return;
+        default: break;
+        }
+    }
+    hipLaunchKernelGGL((k_dense_mv<AT, R, EPI, 0>), g, b, 0, dev->stream, x, W, L.y, K, rows, ns, ea, np);
+}
+
+template <class AT, int R>
+static void launch_mv_epi(candy_hip_device *dev, const DenseLaunch &L, int waves, int nv, const NormPro &np) {
     switch (L.epi) {
-    case EPI_RELU2: hipLaunchKernelGGL((k_dense_mv<AT, R, EPI_RELU2>), g, b, 0, dev->stream, x, W, L.y, K, ns, ea); break;
-    case EPI_CAP: hipLaunchKernelGGL((k_dense_mv<AT, R, EPI_CAP>), g, b, 0, dev->stream, x, W, L.y, K, ns, ea); break;
-    default: hipLaunchKernelGGL((k_dense_mv<AT, R, EPI_NONE>), g, b, 0, dev->stream, x, W, L.y, K, ns, ea); break;
+    case EPI_RELU2: launch_mv_nv<AT, R, EPI_RELU2>(dev, L, waves, nv, np); break;
+    case EPI_CAP: launch_mv_nv<AT, R, EPI_CAP>(dev, L, waves, nv, np); break;
+    default: launch_mv_nv<AT, R, EPI_NONE>(dev, L, waves, nv, np); break;
     }
 }
 
 template <class AT>
-static int launch_mv(candy_hip_device *dev, const DenseLaunch &L) {
-    // enough wavefronts for eight per CU before rows are paired
-    const int64_t waves = 8 * (int64_t)dev->num_cus;
-    if (L.w->rows_pad >= 4 * waves) launch_mv_epi<AT, 4>(dev, L);
-    else if (L.w->rows_pad >= 2 * waves) launch_mv_epi<AT, 2>(dev, L);
-    else launch_mv_epi<AT, 1>(dev, L);
+static int launch_mv(candy_hip_device *dev, const DenseLaunch &L, const MvShape &s, int nv = 0, const NormPro &np = NormPro{}) {
+    switch (s.rows) {
+    case 1: launch_mv_epi<AT, 1>(dev, L, s.waves, nv, np); break;
+    case 2: launch_mv_epi<AT, 2>(dev, L, s.waves, nv, np); break;
+    default: launch_mv_epi<AT, 4>(dev, L, s.waves, nv, np); break;
+    }
     CANDY_LAUNCH_CHECK();
     return CANDY_HIP_OK;
+}
+
+int launch_dense_norm(candy_hip_device *dev, const DenseLaunch &L, const NormArgs &A) {
+    // every workgroup repeats the norms: one per CU, or the launch of their own is the cheaper one
+    const MvShape s = mv_shape(dev, L.n_store);
+    const int per = 256 * s.waves, nv = (int)((L.w->ld + per - 1) / per);
+    if (L.m != 1 || L.f32 || A.rows != 1 || A.y.copies != 1 || A.row_ids || A.x == A.x_out || nv > 2 || L.w->ld > mv_lds_values<bf16>() ||
+        L.n_store > 64 * (int64_t)dev->num_cus)
+        return CANDY_HIP_ERR_UNSUPPORTED;
+    CANDY_REQUIRE(pad64(A.cols) == L.w->ld, "internal: norm and contraction of different widths");
+    if (L.partial) *L.partial = Partial{(const float *)L.y, 1, 0, (int)L.ldy};
+    const NormPro np{A.x, A.y.p, A.post_w, A.post_b, A.step, A.pre_w, A.pre_b, A.x_out, A.mult, A.eps, A.cols};
+    return launch_mv<bf16>(dev, L, s, nv, np);
 }
 
 template <int BM>
@@ -354,7 +487,10 @@ int launch_dense(candy_hip_device *dev, const DenseLaunch &L) {
         L.partial->stride = 0;
         L.partial->ld = (int)L.ldy;
     }
-    if (L.m == 1) return L.f32 ? launch_mv<float>(dev, L) : launch_mv<bf16>(dev, L);
+    if (L.m == 1) {
+        const MvShape s = mv_shape(dev, L.n_store);
+        return L.f32 ? launch_mv<float>(dev, L, s) : launch_mv<bf16>(dev, L, s);
+    }
     if (!L.f32) return L.m <= 64 ? launch_mm<64>(dev, L) : launch_mm<128>(dev, L);
     const dim3 g((unsigned)(w->rows_pad / 64), (unsigned)((L.m + 63) / 64)), b(256);
     CANDY_REQUIRE((L.m + 63) / 64 <= 65535, "prompt too long for one pass");
@@ -373,8 +509,6 @@ int launch_dense(candy_hip_device *dev, const DenseLaunch &L) {
     CANDY_LAUNCH_CHECK();
     return CANDY_HIP_OK;
 }
-
-int launch_dense_norm(candy_hip_device *, const DenseLaunch &, const NormArgs &) { return CANDY_HIP_ERR_UNSUPPORTED; }
 
 // rows ids[i] of a bfloat16 table, widened; an id outside the table raises the handle's fault word and gives zeros
 __global__ __launch_bounds__(256) void k_dense_gather(const bf16 *__restrict__ W, int64_t rows, int64_t ld,

@@ -73,6 +73,13 @@ def test_nil_and_shape_errors_do_not_need_a_device():
     assert b"unknown quantized format" in L.candy_hip_last_error()
     assert L.candy_hip_matmul_f32(None, None, None, None, 1, 0, 1, 1, 0) == 1
     assert b"invalid matrix dimensions" in L.candy_hip_last_error()  # cpu/storage.go:877-879
+    # the other decoder and the generic entry points
+    assert L.candy_hip_suvazen_create(None, None, None, ctypes.byref(out)) == 1
+    assert L.candy_hip_decoder_decode(None, 0, 0, None, None) == 1
+    assert L.candy_hip_decoder_prefill_rows(None, None, 1, 0, None, 0, None) == 1
+    assert L.candy_hip_decoder_free(None) == 0
+    assert L.candy_hip_dense_upload(None, 1, 1, None, ctypes.byref(out)) == 1
+    assert [L.candy_hip_attn_row(d) for d in (0, 1, 32, 33, 80, 128, 129, 256, 257)] == [0, 32, 32, 64, 96, 128, 192, 256, 0]
 
 
 @pytest.mark.skipif(hip.device_count() > 0, reason="only meaningful without a GPU")

@@ -714,6 +714,19 @@ def test_prompt_in_two_chunks_equals_one_pass(dev, case, n, cut):
         a.prefill([], 0)
 
 
+def test_portions_through_the_generic_feed(dev):
+    # Decoder.feed: chosen rows of a prompt pass, single tokens through the decode step, and no rows at all
+    name, cfg, fmts, _, _ = PROMPT_CASES[0]
+    _, a = build(dev, cfg, fmts, seed=13)
+    _, b = build(dev, cfg, fmts, seed=13)
+    tokens = [int(t) for t in np.random.default_rng(15).integers(0, cfg["vocab"], 40)]
+    want = np.stack([a.decode(t, p)[1] for p, t in enumerate(tokens)])
+    got = np.concatenate([b.feed(tokens[:17], 0, [0, 16, 5]), b.feed(tokens[17:18], 17, [0]), b.feed(tokens[18:30], 18, []),
+                          b.feed(tokens[30:], 30, [9])])
+    # the prompt pass and the decode step sum in different orders, and a Q8_0 level that flips for it carries on
+    assert rel(got, want[[0, 16, 5, 17, 39]].astype(np.float64)) <= 5e-3
+
+
 @pytest.mark.parametrize("cut", [20, 77, 128])
 def test_prompt_attention_with_one_and_two_key_tile_groups(dev, cut):
     # The matrix-core kernel's two forms (one group of wavefronts per query tile walking every key tile; two groups
