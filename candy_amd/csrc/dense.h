@@ -47,8 +47,7 @@ struct DenseLaunch {
 };
 int launch_dense(candy_hip_device *dev, const DenseLaunch &L);
 
-// Decode step, one row: the norms in front of a contraction run in its own prologue (layer_norm.hip has the same
-// arithmetic as a launch of its own).  x_out receives the new residual row; it must not be the row that is read.
+// The norms between two sublayers, per row: x + mult * norm(y) + step is the new residual row, out the norm of it.
 struct NormArgs {
     const float *x = nullptr;       // residual rows, ldx apart
     int64_t ldx = 0;
@@ -65,9 +64,10 @@ struct NormArgs {
     int rows = 0, cols = 0;
     const int *row_ids = nullptr;   // optional: row r of the output is made from residual row row_ids[r]
 };
-int launch_norm_chain(candy_hip_device *dev, const NormArgs &A);
+int launch_norm_chain(candy_hip_device *dev, const NormArgs &A);  // layer_norm.hip; x_out may be x
 
-// the bfloat16 contraction of one row with that prologue; CANDY_HIP_ERR_UNSUPPORTED if the row is too wide for it
+// One bfloat16 row: the same norms in the prologue of the contraction that reads them (every workgroup repeats them, so
+// x_out must not be x).  CANDY_HIP_ERR_UNSUPPORTED where two launches are the way.
 int launch_dense_norm(candy_hip_device *dev, const DenseLaunch &L, const NormArgs &A);
 // f32 rows <-> activation rows of `ld` values (zero past cols)
 int launch_to_act(candy_hip_device *dev, bool f32, const float *src, void *dst, int64_t rows, int64_t cols, int64_t ld);
@@ -104,8 +104,5 @@ __device__ __forceinline__ float tanh_fast(float z) {
     const float e = __builtin_amdgcn_exp2f(z * 2.88539008177792681f);  // exp(2z); inf and 0 are fine below
     return 1.0f - 2.0f * __builtin_amdgcn_rcpf(e + 1.0f);
 }
-
-__device__ __forceinline__ float act_load(const float *p) { return *p; }
-__device__ __forceinline__ float act_load(const bf16 *p) { return (float)*p; }
 
 }  // namespace candy

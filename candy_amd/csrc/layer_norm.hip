@@ -3,7 +3,7 @@
 //     x <- x + mult * LN(y) (+ step),   out = LN(x),
 // in one pass over the row.  Everything in f32; `out` is rounded to the activation format on the store.
 // One workgroup per row, the row in registers; mean and variance in two passes over them.
-// (No counterpart in the reference, whose norms are RMSNorm and a layer norm without the chain, reduce.go.)
+// (No counterpart on the reference path this library stands behind, whose norm is RMSNorm, reduce.go:3071-3092.)
 #include <algorithm>
 
 #include "blocks.h"
