@@ -14,14 +14,9 @@
 #include <cmath>
 #include <vector>
 
-#include "blocks.h"
 #include "dense.h"
 
 namespace candy {
-
-constexpr float LOW = -1e30f;      // a running maximum nothing has entered yet
-constexpr float MASKED = -3e38f;   // exp of it is 0 whatever the maximum
-constexpr float LOG2E = 1.44269504088896341f;
 
 int attn_row(int head_dim) {
     for (int r : {32, 64, 96, 128, 192, 256})
@@ -338,17 +333,6 @@ __global__ __launch_bounds__(256, 2) void k_window_attn_prompt(const WindowArgs 
 // splits round robin.  The new token's rows do not go through memory: split 0 rotates and appends them, and its first
 // wavefront attends to them from LDS.
 constexpr int DEC_UNR = 4;
-
-// Sum over groups of LPR neighbouring lanes, in every lane of the group, on the DPP path.
-template <int LPR>
-__device__ __forceinline__ float lanes_sum(float v) {
-    v += dpp_move<0xB1>(v);                       // quad_perm [1,0,3,2]
-    v += dpp_move<0x4E>(v);                       // quad_perm [2,3,0,1]
-    if (LPR >= 8) v += dpp_move<0x141>(v);        // row_half_mirror
-    if (LPR >= 16) v += dpp_move<0x140>(v);       // row_mirror
-    if (LPR >= 32) v += __shfl_xor(v, 16, 64);
-    return v;
-}
 
 template <int LPR> constexpr int dec_batch() { return 4 * (64 / LPR) * DEC_UNR; }
 

@@ -1,5 +1,5 @@
 // What every decoder of the library shares: the KV cache, the captured decode step and its replay, the prompt pass
-// around a model's layers, greedy generation.  A model (llama.hip, suvazen.hip) derives from candy_hip_decoder and
+// around a model's layers, greedy generation.  A model (llama.hip, suvazen.hip, gulisun.hip) derives from candy_hip_decoder and
 // supplies the layers; positions, tokens, logits, graphs and the cache are handled here.  (candy has no model code:
 // no counterpart in the reference.)
 #pragma once
@@ -10,8 +10,8 @@
 
 namespace candy {
 
-// Keys and values of all layers in two allocations.  Layer l's part is [kv heads][max_pos][row width]; the widths may
-// differ from layer to layer.  A row is written when its position is fed and read only by later positions of the same
+// Keys and values of all layers in two allocations, or in one where a row serves as both (latent attention).  Layer l's
+// part is [kv heads][max_pos][row width]; the widths may differ from layer to layer.  A row is written when its position is fed and read only by later positions of the same
 // sequence, so a sequence that starts over at position 0 needs no clearing.
 struct KvCache {
     struct Layer {
@@ -22,6 +22,7 @@ struct KvCache {
     int max_pos = 0, elem_bytes = 4;
     std::vector<Layer> layers;
     size_t values = 0;                // per array
+    bool one_array = false;           // no separate values: v stays null
     void *k = nullptr, *v = nullptr;
 
     void add_layer(int n_kv_heads, int row) {
@@ -38,6 +39,23 @@ struct KvCache {
     size_t bytes() const { return values * (size_t)elem_bytes; }
 };
 
+// State of the recurrent layers, f32, one part per layer in one allocation.  It belongs to the sequence being fed and
+// stands behind position next - 1; layers take position 0 as a fresh start whatever the state holds, so a sequence that
+// starts over needs no clearing, but positions can only be fed in order.
+struct RecurrentState {
+    std::vector<size_t> offset;
+    size_t floats = 0;
+    float *data = nullptr;
+    int next = 0;                     // -1: a call was cut short, only position 0 makes sense
+
+    int add_layer(size_t n) {
+        offset.push_back(floats);
+        floats += n;
+        return (int)offset.size() - 1;
+    }
+    float *of(int l) const { return data + offset[(size_t)l]; }
+};
+
 }  // namespace candy
 
 struct candy_hip_decoder {
@@ -45,6 +63,7 @@ struct candy_hip_decoder {
     int width = 0, vocab = 0, max_pos = 0;
     int width_pad = 0;                          // floats between rows of the residual stream
     candy::KvCache cache;
+    candy::RecurrentState state;                // empty for models without recurrent layers
     float *h = nullptr;                         // residual stream of the token being decoded
     float *logits = nullptr;
     unsigned long long *next_key = nullptr;     // greedy token of the last step as k_argmax_key leaves it; zero before a step

@@ -24,12 +24,14 @@ __global__ void k_chain_step(int *pos_dst, int pos, int64_t *tok_dst, unsigned l
 int decoder_init(candy_hip_decoder *m) {
     int rc = CANDY_HIP_OK;
     uint8_t *k = nullptr, *v = nullptr;
-    if (!rc) rc = decoder_alloc(m, &k, m->cache.bytes());
-    if (!rc) rc = decoder_alloc(m, &v, m->cache.bytes());
+    if (!rc && m->cache.bytes()) rc = decoder_alloc(m, &k, m->cache.bytes());
+    if (!rc && m->cache.bytes() && !m->cache.one_array) rc = decoder_alloc(m, &v, m->cache.bytes());
     m->cache.k = k;
     m->cache.v = v;
-    if (!rc) rc = candy_hip_zero(m->dev, k, m->cache.bytes());
-    if (!rc) rc = candy_hip_zero(m->dev, v, m->cache.bytes());
+    if (!rc && k) rc = candy_hip_zero(m->dev, k, m->cache.bytes());
+    if (!rc && v) rc = candy_hip_zero(m->dev, v, m->cache.bytes());
+    if (!rc && m->state.floats) rc = decoder_alloc(m, &m->state.data, m->state.floats);
+    if (!rc && m->state.floats) rc = candy_hip_zero(m->dev, m->state.data, m->state.floats * sizeof(float));
     if (!rc) rc = decoder_alloc(m, &m->h, (size_t)m->width_pad);
     if (!rc) rc = candy_hip_zero(m->dev, m->h, (size_t)m->width_pad * sizeof(float));  // what pads the row stays zero
     if (!rc) rc = decoder_alloc(m, &m->logits, (size_t)m->vocab + 4);  // the argmax kernel reads whole 16-byte pieces
@@ -55,11 +57,19 @@ int candy_hip_decoder::enqueue_head_rows(const int32_t *rows, int n_rows, float 
     return CANDY_HIP_OK;
 }
 
+// Whether a call may feed position pos: recurrent state stands behind one position only.
+static int check_order(const candy_hip_decoder *m, int32_t pos) {
+    CANDY_REQUIRE(!m->state.floats || pos == 0 || pos == m->state.next, "position %d out of order: the recurrent state stands in front of %d",
+                  pos, m->state.next);
+    return CANDY_HIP_OK;
+}
+
 // chain_to: null, or where the token chosen by the previous step is recorded while it becomes this step's input
 static int decoder_step(candy_hip_decoder *m, int32_t pos, int64_t token, const float *dev_hidden,
                         const float **dev_logits, int32_t *next_token, int32_t *chain_to = nullptr) {
     candy_hip_device *dev = m->dev;
     int rc;
+    m->state.next = -1;
     if (chain_to)
         hipLaunchKernelGGL(k_chain_step, dim3(1), dim3(1), 0, dev->stream, m->d_pos, (int)pos, m->tok_id, m->next_key, chain_to);
     else
@@ -96,6 +106,7 @@ static int decoder_step(candy_hip_decoder *m, int32_t pos, int64_t token, const 
         (void)m->reset_step();  // see above
         return rc;
     }
+    m->state.next = pos + 1;
     if (dev_logits) *dev_logits = m->logits;
     if (next_token) {
         unsigned long long key = 0;
@@ -118,6 +129,7 @@ static int decoder_feed(candy_hip_decoder *m, const int32_t *tokens, int32_t n_t
         ids[(size_t)i] = tokens[i];
     }
     if (int rc = m->check_complete()) return rc;
+    if (int rc = check_order(m, pos0)) return rc;
     if (int rc = use_device(m->dev)) return rc;
     if (n_tokens > m->prompt_cap) {
         CANDY_HIP_TRY(hipStreamSynchronize(m->dev->stream));
@@ -129,7 +141,10 @@ static int decoder_feed(candy_hip_decoder *m, const int32_t *tokens, int32_t n_t
         m->prompt_cap = n_tokens;
     }
     if (int rc = candy_hip_h2d(m->dev, m->prompt_ids, ids.data(), ids.size() * sizeof(int64_t))) return rc;
-    return m->enqueue_prompt(n_tokens, pos0);
+    m->state.next = -1;
+    if (int rc = m->enqueue_prompt(n_tokens, pos0)) return rc;
+    m->state.next = pos0 + n_tokens;
+    return CANDY_HIP_OK;
 }
 
 extern "C" {
@@ -220,6 +235,7 @@ int candy_hip_decoder_decode_hidden(candy_hip_decoder *m, const float *dev_hidde
     CANDY_REQUIRE(m && dev_hidden, "nil argument");
     CANDY_REQUIRE(pos >= 0 && pos < m->max_pos, "position %d outside the cache (max_pos %d)", pos, m->max_pos);
     if (int rc = m->check_complete()) return rc;
+    if (int rc = check_order(m, pos)) return rc;
     if (int rc = use_device(m->dev)) return rc;
     return decoder_step(m, pos, -1, dev_hidden, dev_logits, next_token);
 }
@@ -231,6 +247,7 @@ int candy_hip_decoder_decode(candy_hip_decoder *m, int32_t token, int32_t pos, c
     CANDY_REQUIRE(token >= 0 && token < m->vocab, "token %d outside the vocabulary", token);
     CANDY_REQUIRE(pos >= 0 && pos < m->max_pos, "position %d outside the cache (max_pos %d)", pos, m->max_pos);
     if (int rc = m->check_complete()) return rc;
+    if (int rc = check_order(m, pos)) return rc;
     if (int rc = use_device(m->dev)) return rc;
     return decoder_step(m, pos, token, nullptr, dev_logits, next_token);
 }
@@ -243,6 +260,7 @@ int candy_hip_decoder_generate(candy_hip_decoder *m, int32_t token, int32_t pos,
     CANDY_REQUIRE(pos >= 0 && (int64_t)pos + n_steps <= m->max_pos, "positions %d .. %lld outside the cache (max_pos %d)",
                   pos, (long long)pos + n_steps - 1, m->max_pos);
     if (int rc = m->check_complete()) return rc;
+    if (int rc = check_order(m, pos)) return rc;
     if (int rc = use_device(m->dev)) return rc;
     int32_t *list = nullptr;  // one slot per step; slot i takes the token step i chose
     if (int rc = candy_hip_alloc(m->dev, (size_t)(n_steps + 1) * sizeof(int32_t), (void **)&list)) return rc;

@@ -4,16 +4,18 @@
 //   k_dense_mm      prompt batches, bfloat16 activations: v_mfma_f32_16x16x32_bf16 over LDS tiles filled by direct
 //                   global-to-LDS loads, two stages; optionally split along K
 //   k_dense_mm_f32  prompt batches, f32 activations: v_mfma_f32_16x16x4_f32, weights widened exactly
+// Prompt batches also come with block-diagonal weights, and with their rows dealt to experts (GroupedRows).
 // Weights are stored with both sides padded to multiples of 64 by zeros, so no kernel has a ragged edge in K, and the
 // padded rows come out as epilogue(0) = 0.  (No counterpart in the reference, which has no bfloat16.)
 #include <algorithm>
 
-#include "blocks.h"
 #include "dense.h"
 
 namespace candy {
 
-constexpr int EPI_NONE = CANDY_HIP_EPI_NONE, EPI_RELU2 = CANDY_HIP_EPI_SQUARED_RELU, EPI_CAP = CANDY_HIP_EPI_SOFTCAP;
+constexpr int EPI_NONE = CANDY_HIP_EPI_NONE, EPI_RELU2 = CANDY_HIP_EPI_SQUARED_RELU, EPI_CAP = CANDY_HIP_EPI_SOFTCAP,
+              EPI_ACT = CANDY_HIP_EPI_ACT;
+constexpr bool to_act(int epi) { return epi == EPI_RELU2 || epi == EPI_ACT; }  // the result is in the activation format
 
 struct EpiArgs {
     float scale, cap;
@@ -32,27 +34,13 @@ __device__ __forceinline__ float epilogue(float z, const EpiArgs &e) {
     return z;
 }
 
-__device__ __forceinline__ void widen8(u32x4v v, float (&f)[8]) {
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-        f[2 * i] = __uint_as_float(v[i] << 16);
-        f[2 * i + 1] = __uint_as_float(v[i] & 0xFFFF0000u);
-    }
-}
-__device__ __forceinline__ void lds8(const bf16 *p, float (&f)[8]) { widen8(*(const u32x4v *)p, f); }
-__device__ __forceinline__ void lds8(const float *p, float (&f)[8]) {
-    const f32x4 a = *(const f32x4 *)p, b = *(const f32x4 *)(p + 4);
-#pragma unroll
-    for (int i = 0; i < 4; ++i) { f[i] = a[i]; f[4 + i] = b[i]; }
-}
-
 // ------------------------------------------------------------------ one row
 // The norms in front of the contraction (launch_norm_chain's arithmetic), for a kernel that runs them in its prologue.
 struct NormPro {
     const float *x, *y, *post_w, *post_b, *step, *pre_w, *pre_b;
     float *x_out;
     float mult, eps;
-    int cols;
+    int cols, rms;
 };
 
 __device__ __forceinline__ float pro_sum(float v, float *red) {
@@ -128,21 +116,26 @@ __global__ __launch_bounds__(1024) void k_dense_mv(const AT *__restrict__ x, con
             for (int i = 0; i < NV; ++i) d[i] = (tid + threads * i) * 4 < K ? *(const f32x4 *)(p + (tid + threads * i) * 4) : zero;
         };
         f32x4 wv[NV], bv[NV], pw[NV], pb[NV];
+#pragma unroll
+        for (int i = 0; i < NV; ++i) bv[i] = pb[i] = zero;
         load(np.x, xv);
         if (np.y) {
             load(np.y, yv4);
             load(np.post_w, pw);
-            load(np.post_b, pb);
+            if (np.post_b) load(np.post_b, pb);
         }
-        load(np.pre_w, wv);
-        load(np.pre_b, bv);
+        if (np.pre_w) load(np.pre_w, wv);
+        if (np.pre_b) load(np.pre_b, bv);
         fetch(wa, 0);
         const float inv_n = 1.0f / (float)np.cols;
         auto normalize = [&](f32x4 (&d)[NV], const f32x4 (&w)[NV], const f32x4 (&b)[NV]) __attribute__((always_inline)) {
-            float s = 0.0f;
+            float mean = 0.0f;
+            if (!np.rms) {
+                float s = 0.0f;
 #pragma unroll
-            for (int i = 0; i < NV; ++i) s += (d[i][0] + d[i][1]) + (d[i][2] + d[i][3]);
-            const float mean = pro_sum(s, red) * inv_n;
+                for (int i = 0; i < NV; ++i) s += (d[i][0] + d[i][1]) + (d[i][2] + d[i][3]);
+                mean = pro_sum(s, red) * inv_n;
+            }
             float q = 0.0f;
 #pragma unroll
             for (int i = 0; i < NV; ++i)
@@ -172,7 +165,7 @@ __global__ __launch_bounds__(1024) void k_dense_mv(const AT *__restrict__ x, con
             for (int i = 0; i < NV; ++i)
                 if ((tid + threads * i) * 4 < K) *(f32x4 *)(np.x_out + (tid + threads * i) * 4) = xv[i];
         }
-        normalize(xv, wv, bv);
+        if (np.pre_w) normalize(xv, wv, bv);
         typedef AT at4 __attribute__((ext_vector_type(4)));
         const int n = (K + STEP - 1) / STEP * STEP;
 #pragma unroll
@@ -199,7 +192,7 @@ __global__ __launch_bounds__(1024) void k_dense_mv(const AT *__restrict__ x, con
     }
     if (lane < R && row0 + lane < n_store) {
         const float z = epilogue<EPI>(mine, ea);
-        if (EPI == EPI_RELU2) ((AT *)yv)[row0 + lane] = (AT)z;
+        if (to_act(EPI)) ((AT *)yv)[row0 + lane] = (AT)z;
         else ((float *)yv)[row0 + lane] = z;
     }
 }
@@ -208,10 +201,12 @@ __global__ __launch_bounds__(1024) void k_dense_mv(const AT *__restrict__ x, con
 // Tile: BN = 128 weight rows x BM activation rows, 64 values of K per stage.  A row of a stage is 128 bytes = eight
 // 16-byte chunks; chunk c of row r sits in slot c ^ ((r >> 1) & 7), so that the 16 rows a fragment read touches spread
 // over all banks.  A direct load writes 64 consecutive 16-byte slots, so the permutation is in the addresses it reads.
-template <int BM, int EPI>
+// GROUPED: the row tiles come from a list in device memory (of BM rows at most each), one expert's weights per tile.
+template <int BM, int EPI, bool GROUPED>
 __global__ __launch_bounds__(256, 2) void k_dense_mm(const bf16 *__restrict__ W, const bf16 *__restrict__ X, void *__restrict__ yv,
                                                      int M, int Np, int ld, int ldx, int k_slice, int64_t ldy, int n_store,
-                                                     size_t split_stride, int m_tiles, int n_tiles, const EpiArgs ea) {
+                                                     size_t split_stride, int m_tiles, int n_tiles, int block_rows, const EpiArgs ea,
+                                                     const GroupedRows gr) {
     constexpr int BN = 128, BK = 64, ROWS = BN + BM, LOADS = ROWS / 32;
     constexpr int TN = 4, TM = BM / 32;
     __shared__ __align__(16) u32x4v s[2][ROWS * 8];
@@ -219,20 +214,34 @@ __global__ __launch_bounds__(256, 2) void k_dense_mm(const bf16 *__restrict__ W,
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     // each XCD takes a run of neighbouring tiles (workgroups are dealt to the XCDs round robin); the activation tiles of
     // one weight tile are neighbours
+    if (GROUPED) m_tiles = *gr.n_tiles;
     const int total = m_tiles * n_tiles;
     int t = blockIdx.x;
+    if (GROUPED && t >= total) return;
     {
         const int per = total >> 3, full = per << 3;
         if (t < full) t = (t & 7) * per + (t >> 3);
     }
-    const int m0 = (t % m_tiles) * BM, n0 = (t / m_tiles) * BN;
+    const int n0 = (t / m_tiles) * BN;
+    int m0 = (t % m_tiles) * BM;
+    const int *perm = nullptr;
+    if (GROUPED) {
+        const GroupTile tile = gr.tiles[t % m_tiles];
+        W += (size_t)tile.expert * Np * ld;
+        perm = gr.perm + tile.first;
+        M = tile.count;
+        m0 = 0;
+    }
+    if (block_rows) X += (size_t)(n0 / block_rows) * ld;
     const int kbeg = blockIdx.y * k_slice, kend = min(kbeg + k_slice, ld);
     const bf16 *src[LOADS];
 #pragma unroll
     for (int i = 0; i < LOADS; ++i) {
         const int r = (wave + 4 * i) * 8 + (lane >> 3);
         const int c = (lane & 7) ^ ((r >> 1) & 7);
-        src[i] = (r < BN ? W + (size_t)min(n0 + r, Np - 1) * ld : X + (size_t)min(m0 + r - BN, M - 1) * ldx) + kbeg + c * 8;
+        int xr = min(m0 + max(r - BN, 0), M - 1);
+        if (GROUPED) xr = perm[xr] / gr.x_div;
+        src[i] = (r < BN ? W + (size_t)min(n0 + r, Np - 1) * ld : X + (size_t)xr * ldx) + kbeg + c * 8;
     }
     auto load = [&](int stage) __attribute__((always_inline)) {
 #pragma unroll
@@ -276,15 +285,16 @@ __global__ __launch_bounds__(256, 2) void k_dense_mm(const bf16 *__restrict__ W,
     // C layout: column r16 is the activation row, rows 4g .. 4g+3 are four neighbouring outputs of it
 #pragma unroll
     for (int j = 0; j < TM; ++j) {
-        const int m = m0 + wm - BN + j * 16 + r16;
+        int m = m0 + wm - BN + j * 16 + r16;
         if (m >= M) continue;
+        if (GROUPED) m = perm[m];
 #pragma unroll
         for (int i = 0; i < TN; ++i) {
             const int n = n0 + wn + i * 16 + 4 * g;
             f32x4 z = acc[i][j];
 #pragma unroll
             for (int e = 0; e < 4; ++e) z[e] = epilogue<EPI>(z[e], ea);
-            if (EPI == EPI_RELU2) {
+            if (to_act(EPI)) {
                 if (n < n_store) *(bf16x4 *)((bf16 *)yv + (size_t)m * ldy + n) = __builtin_convertvector(z, bf16x4);
             } else if (EPI == EPI_NONE) {
                 float *y = (float *)yv + blockIdx.y * split_stride + (size_t)m * ldy + n;
@@ -303,13 +313,25 @@ __global__ __launch_bounds__(256, 2) void k_dense_mm(const bf16 *__restrict__ W,
 }
 
 // ------------------------------------------------------------------ prompt batches, f32 activations
-template <int EPI>
+template <int EPI, bool GROUPED>
 __global__ __launch_bounds__(256) void k_dense_mm_f32(const bf16 *__restrict__ W, const float *__restrict__ X, float *__restrict__ yv,
-                                                      int M, int ld, int ldx, int64_t ldy, int n_store, const EpiArgs ea) {
+                                                      int M, int ld, int ldx, int64_t ldy, int n_store, int block_rows,
+                                                      const EpiArgs ea, const GroupedRows gr) {
     constexpr int B = 64, BK = 32, P = BK + 4;
     __shared__ __align__(16) float sw[B * P], sx[B * P];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-    const int n0 = blockIdx.x * B, m0 = blockIdx.y * B;
+    const int n0 = blockIdx.x * B;
+    int m0 = blockIdx.y * B;
+    const int *perm = nullptr;
+    if (GROUPED) {
+        if ((int)blockIdx.y >= *gr.n_tiles) return;
+        const GroupTile tile = gr.tiles[blockIdx.y];
+        W += (size_t)tile.expert * gr.expert_rows * ld;
+        perm = gr.perm + tile.first;
+        M = tile.count;
+        m0 = 0;
+    }
+    if (block_rows) X += (size_t)(n0 / block_rows) * ld;
     const int r16 = lane & 15, g = lane >> 4;
     const int wn = (wave >> 1) * 32, wm = (wave & 1) * 32;
     f32x4 acc[2][2];
@@ -318,10 +340,12 @@ __global__ __launch_bounds__(256) void k_dense_mm_f32(const bf16 *__restrict__ W
 #pragma unroll
         for (int j = 0; j < 2; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
     const int lr = tid >> 2, lc = (tid & 3) * 8;  // a row of the stage, 8 of its 32 values
+    int xr = min(m0 + lr, M - 1);
+    if (GROUPED) xr = perm[xr] / gr.x_div;
     for (int k0 = 0; k0 < ld; k0 += BK) {
         float wf[8], xf[8];
         widen8(*(const u32x4v *)(W + (size_t)(n0 + lr) * ld + k0 + lc), wf);
-        lds8(X + (size_t)min(m0 + lr, M - 1) * ldx + k0 + lc, xf);
+        lds8(X + (size_t)xr * ldx + k0 + lc, xf);
         __syncthreads();
 #pragma unroll
         for (int e = 0; e < 8; ++e) {
@@ -345,8 +369,9 @@ __global__ __launch_bounds__(256) void k_dense_mm_f32(const bf16 *__restrict__ W
     }
 #pragma unroll
     for (int j = 0; j < 2; ++j) {
-        const int m = m0 + wm + j * 16 + r16;
+        int m = m0 + wm + j * 16 + r16;
         if (m >= M) continue;
+        if (GROUPED) m = perm[m];
 #pragma unroll
         for (int i = 0; i < 2; ++i)
 #pragma unroll
@@ -358,13 +383,9 @@ __global__ __launch_bounds__(256) void k_dense_mm_f32(const bf16 *__restrict__ W
 }
 
 // ------------------------------------------------------------------ launches
-struct MvShape {
-    int waves, rows;  // wavefronts per workgroup, weight rows per wavefront
-};
-
 // Rows over wavefronts: with up to 64 rows per CU one workgroup per CU takes them all, its shape the one that leaves the
 // fewest slots empty (the more wavefronts the better, from eight on); longer weights take many workgroups of 8 x 4.
-static MvShape mv_shape(const candy_hip_device *dev, int64_t rows) {
+MvShape mv_shape(const candy_hip_device *dev, int64_t rows) {
     const int64_t per_cu = (rows + dev->num_cus - 1) / dev->num_cus;
     if (per_cu > 64) return {8, 4};
     if (per_cu <= 8) return {8, 1};
@@ -388,7 +409,7 @@ static void launch_mv_nv(candy_hip_device *dev, const DenseLaunch &L, int waves,
     const AT *x = (const AT *)L.x;
     const bf16 *W = (const bf16 *)L.w->data;
     const int K = (int)L.w->ld, rows = (int)L.w->rows_pad, ns = (int)L.n_store;
-    if constexpr (sizeof(AT) == 2) {
+    if constexpr (sizeof(AT) == 2 || (R == 1 && EPI == EPI_NONE)) {
         switch (nv) {
         case 1: hipLaunchKernelGGL((k_dense_mv<AT, R, EPI, 1>), g, b, 0, dev->stream, x, W, L.y, K, rows, ns, ea, np); return;
         case 2: hipLaunchKernelGGL((k_dense_mv<AT, R, EPI, 2>), g, b, 0, dev->stream, x, W, L.y, K, rows, ns, ea, np); return;
@@ -403,6 +424,7 @@ static void launch_mv_epi(candy_hip_device *dev, const DenseLaunch &L, int waves
     switch (L.epi) {
     case EPI_RELU2: launch_mv_nv<AT, R, EPI_RELU2>(dev, L, waves, nv, np); break;
     case EPI_CAP: launch_mv_nv<AT, R, EPI_CAP>(dev, L, waves, nv, np); break;
+    case EPI_ACT: launch_mv_nv<AT, R, EPI_ACT>(dev, L, waves, nv, np); break;
     default: launch_mv_nv<AT, R, EPI_NONE>(dev, L, waves, nv, np); break;
     }
 }
@@ -422,13 +444,13 @@ int launch_dense_norm(candy_hip_device *dev, const DenseLaunch &L, const NormArg
     // every workgroup repeats the norms: one per CU, or the launch of their own is the cheaper one
     const MvShape s = mv_shape(dev, L.n_store);
     const int per = 256 * s.waves, nv = (int)((L.w->ld + per - 1) / per);
-    if (L.m != 1 || L.f32 || A.rows != 1 || A.y.copies != 1 || A.row_ids || A.x == A.x_out || nv > 2 || L.w->ld > mv_lds_values<bf16>() ||
-        L.n_store > 64 * (int64_t)dev->num_cus)
+    if (L.m != 1 || (L.f32 && (s.rows != 1 || L.epi != EPI_NONE)) || A.rows != 1 || A.y.copies != 1 || A.slots || A.row_ids ||
+        A.x == A.x_out || nv > 2 || L.w->ld > (L.f32 ? mv_lds_values<float>() : mv_lds_values<bf16>()) || L.n_store > 64 * (int64_t)dev->num_cus)
         return CANDY_HIP_ERR_UNSUPPORTED;
     CANDY_REQUIRE(pad64(A.cols) == L.w->ld, "internal: norm and contraction of different widths");
     if (L.partial) *L.partial = Partial{(const float *)L.y, 1, 0, (int)L.ldy};
-    const NormPro np{A.x, A.y.p, A.post_w, A.post_b, A.step, A.pre_w, A.pre_b, A.x_out, A.mult, A.eps, A.cols};
-    return launch_mv<bf16>(dev, L, s, nv, np);
+    const NormPro np{A.x, A.y.p, A.post_w, A.post_b, A.step, A.pre_w, A.pre_b, A.x_out, A.mult, A.eps, A.cols, A.rms};
+    return L.f32 ? launch_mv<float>(dev, L, s, nv, np) : launch_mv<bf16>(dev, L, s, nv, np);
 }
 
 template <int BM>
@@ -463,14 +485,35 @@ static int launch_mm(candy_hip_device *dev, const DenseLaunch &L) {
     const EpiArgs ea{L.scale, L.cap};
     const bf16 *W = (const bf16 *)L.w->data, *X = (const bf16 *)L.x;
 #define CANDY_MM(EPI)                                                                                                     \
-    hipLaunchKernelGGL((k_dense_mm<BM, EPI>), g, b, 0, dev->stream, W, X, y, L.m, (int)L.w->rows_pad, K, (int)L.ldx, k_slice, \
-                       ldy, (int)n_store, stride, m_tiles, n_tiles, ea)
+    hipLaunchKernelGGL((k_dense_mm<BM, EPI, false>), g, b, 0, dev->stream, W, X, y, L.m, (int)L.w->rows_pad, K, (int)L.ldx,   \
+                       k_slice, ldy, (int)n_store, stride, m_tiles, n_tiles, L.block_rows, ea, GroupedRows{})
     switch (L.epi) {
     case EPI_RELU2: CANDY_MM(EPI_RELU2); break;
     case EPI_CAP: CANDY_MM(EPI_CAP); break;
+    case EPI_ACT: CANDY_MM(EPI_ACT); break;
     default: CANDY_MM(EPI_NONE); break;
     }
 #undef CANDY_MM
+    CANDY_LAUNCH_CHECK();
+    return CANDY_HIP_OK;
+}
+
+// Rows dealt to experts: the grid has room for max_tiles row tiles, workgroups past the list's end leave at once.
+template <int BM>
+static int launch_mm_grouped(candy_hip_device *dev, const DenseLaunch &L) {
+    const GroupedRows &gr = *L.group;
+    const int n_tiles = (gr.expert_rows + 127) / 128, K = (int)L.w->ld;
+    const int64_t tiles = (int64_t)gr.max_tiles * n_tiles;
+    CANDY_REQUIRE(tiles <= 0x7FFFFFFF, "matrix too large");
+    const dim3 g((unsigned)tiles), b(256);
+    const EpiArgs ea{L.scale, L.cap};
+    const bf16 *W = (const bf16 *)L.w->data, *X = (const bf16 *)L.x;
+#define CANDY_MMG(EPI)                                                                                                       \
+    hipLaunchKernelGGL((k_dense_mm<BM, EPI, true>), g, b, 0, dev->stream, W, X, L.y, L.m, gr.expert_rows, K, (int)L.ldx, K,  \
+                       L.ldy, (int)L.n_store, (size_t)0, 0, n_tiles, 0, ea, gr)
+    if (L.epi == EPI_RELU2) CANDY_MMG(EPI_RELU2);
+    else CANDY_MMG(EPI_NONE);
+#undef CANDY_MMG
     CANDY_LAUNCH_CHECK();
     return CANDY_HIP_OK;
 }
@@ -480,40 +523,57 @@ int launch_dense(candy_hip_device *dev, const DenseLaunch &L) {
     CANDY_REQUIRE(L.m > 0 && w->rows_pad <= 0x7FFFFFFF && w->ld <= 0x7FFFFFFF && L.ldx >= w->ld && L.ldx <= 0x7FFFFFFF,
                   "internal: dense contraction of a shape the kernels do not take");
     CANDY_REQUIRE(L.n_store <= w->rows_pad && L.ldy >= L.n_store, "internal: dense output row too short");
-    CANDY_REQUIRE(L.epi != EPI_RELU2 || (L.n_store == w->rows_pad && (L.ldy & 63) == 0), "internal: activation rows must be padded");
+    const int64_t out_rows = L.group ? L.group->expert_rows : w->rows_pad;
+    CANDY_REQUIRE(!to_act(L.epi) || (L.n_store == out_rows && (L.ldy & 63) == 0), "internal: activation rows must be padded");
+    CANDY_REQUIRE(L.block_rows == 0 || (!L.partial && L.block_rows % 128 == 0 && w->rows_pad % L.block_rows == 0 &&
+                                        L.ldx >= w->rows_pad / L.block_rows * w->ld), "internal: block-diagonal contraction");
+    if (L.group) {
+        CANDY_REQUIRE((L.epi == EPI_NONE || L.epi == EPI_RELU2) && !L.partial && !L.block_rows && L.group->expert_rows % 64 == 0 &&
+                          w->rows % L.group->expert_rows == 0 && L.group->max_tiles <= 65535,
+                      "internal: grouped contraction");
+        if (!L.f32 && L.group->tile_rows == 128) return launch_mm_grouped<128>(dev, L);
+        CANDY_REQUIRE(L.group->tile_rows == 64, "internal: row tiles of 64");
+        if (!L.f32) return launch_mm_grouped<64>(dev, L);
+    }
     if (L.partial) {
         L.partial->p = (const float *)L.y;
         L.partial->copies = 1;
         L.partial->stride = 0;
         L.partial->ld = (int)L.ldy;
     }
-    if (L.m == 1) {
+    if (L.m == 1 && !L.group && !L.block_rows) {
         const MvShape s = mv_shape(dev, L.n_store);
         return L.f32 ? launch_mv<float>(dev, L, s) : launch_mv<bf16>(dev, L, s);
     }
     if (!L.f32) return L.m <= 64 ? launch_mm<64>(dev, L) : launch_mm<128>(dev, L);
-    const dim3 g((unsigned)(w->rows_pad / 64), (unsigned)((L.m + 63) / 64)), b(256);
+    const dim3 g((unsigned)(out_rows / 64), (unsigned)(L.group ? L.group->max_tiles : (L.m + 63) / 64)), b(256);
     CANDY_REQUIRE((L.m + 63) / 64 <= 65535, "prompt too long for one pass");
     const EpiArgs ea{L.scale, L.cap};
     const bf16 *W = (const bf16 *)w->data;
     const float *X = (const float *)L.x;
 #define CANDY_MM32(EPI)                                                                                                 \
-    hipLaunchKernelGGL((k_dense_mm_f32<EPI>), g, b, 0, dev->stream, W, X, (float *)L.y, L.m, (int)w->ld, (int)L.ldx, L.ldy, \
-                       (int)L.n_store, ea)
+    do {                                                                                                                \
+        if (L.group)                                                                                                    \
+            hipLaunchKernelGGL((k_dense_mm_f32<EPI, true>), g, b, 0, dev->stream, W, X, (float *)L.y, L.m, (int)w->ld,  \
+                               (int)L.ldx, L.ldy, (int)L.n_store, 0, ea, *L.group);                                     \
+        else                                                                                                            \
+            hipLaunchKernelGGL((k_dense_mm_f32<EPI, false>), g, b, 0, dev->stream, W, X, (float *)L.y, L.m, (int)w->ld, \
+                               (int)L.ldx, L.ldy, (int)L.n_store, L.block_rows, ea, GroupedRows{});                     \
+    } while (0)
     switch (L.epi) {
     case EPI_RELU2: CANDY_MM32(EPI_RELU2); break;
     case EPI_CAP: CANDY_MM32(EPI_CAP); break;
-    default: CANDY_MM32(EPI_NONE); break;
+    default: CANDY_MM32(EPI_NONE); break;  // ACT: f32 is the activation format
     }
 #undef CANDY_MM32
     CANDY_LAUNCH_CHECK();
     return CANDY_HIP_OK;
 }
 
-// rows ids[i] of a bfloat16 table, widened; an id outside the table raises the handle's fault word and gives zeros
+// rows ids[i] of a bfloat16 table, widened and scaled; an id outside the table raises the handle's fault word and gives zeros
 __global__ __launch_bounds__(256) void k_dense_gather(const bf16 *__restrict__ W, int64_t rows, int64_t ld,
                                                       const int64_t *__restrict__ ids, float *__restrict__ out, int64_t ldo,
-                                                      int *fault) {
+                                                      float scale, int *fault) {
     const int64_t id = ids[blockIdx.y];
     const int64_t c = ((int64_t)blockIdx.x * 256 + threadIdx.x) * 8;
     if (c >= ld) return;
@@ -521,15 +581,16 @@ __global__ __launch_bounds__(256) void k_dense_gather(const bf16 *__restrict__ W
     if (id >= 0 && id < rows) widen8(*(const u32x4v *)(W + id * ld + c), f);
     else if (c == 0) *fault = 1;
     float *o = out + (int64_t)blockIdx.y * ldo + c;
-    *(f32x4 *)o = f32x4{f[0], f[1], f[2], f[3]};
-    *(f32x4 *)(o + 4) = f32x4{f[4], f[5], f[6], f[7]};
+    *(f32x4 *)o = f32x4{f[0], f[1], f[2], f[3]} * scale;
+    *(f32x4 *)(o + 4) = f32x4{f[4], f[5], f[6], f[7]} * scale;
 }
 
-int launch_dense_gather(candy_hip_device *dev, const candy_hip_dense *w, const int64_t *ids, int64_t n, float *out, int64_t ldo) {
+int launch_dense_gather(candy_hip_device *dev, const candy_hip_dense *w, const int64_t *ids, int64_t n, float *out, int64_t ldo,
+                        float scale) {
     for (int64_t i0 = 0; i0 < n; i0 += 65535) {
         const int64_t part = std::min<int64_t>(n - i0, 65535);
         hipLaunchKernelGGL(k_dense_gather, dim3((unsigned)((w->ld / 8 + 255) / 256), (unsigned)part), dim3(256), 0, dev->stream,
-                           (const bf16 *)w->data, w->rows, w->ld, ids + i0, out + i0 * ldo, ldo, dev->fault);
+                           (const bf16 *)w->data, w->rows, w->ld, ids + i0, out + i0 * ldo, ldo, scale, dev->fault);
         CANDY_LAUNCH_CHECK();
     }
     return CANDY_HIP_OK;
@@ -625,7 +686,7 @@ int candy_hip_dense_matmul(candy_hip_device *dev, const candy_hip_dense *w, cons
     CANDY_REQUIRE(dev && w->dev == dev, "rhs storage must live on the same HIP device");
     CANDY_REQUIRE(m >= 0 && m <= 1 << 20, "invalid matrix dimensions");
     CANDY_REQUIRE(act == CANDY_HIP_ACT_BF16 || act == CANDY_HIP_ACT_F32, "unknown activation format %d", act);
-    CANDY_REQUIRE(epilogue >= EPI_NONE && epilogue <= EPI_CAP, "unknown epilogue %d", epilogue);
+    CANDY_REQUIRE(epilogue >= EPI_NONE && epilogue <= EPI_ACT, "unknown epilogue %d", epilogue);
     if (m == 0) return CANDY_HIP_OK;
     CANDY_REQUIRE(dev_x && dev_y, "nil pointer");
     if (int rc = use_device(dev)) return rc;
@@ -636,7 +697,7 @@ int candy_hip_dense_matmul(candy_hip_device *dev, const candy_hip_dense *w, cons
     if (int rc = launch_to_act(dev, f32, dev_x, ws, m, w->cols, w->ld)) return rc;
     DenseLaunch L;
     L.w = w; L.x = ws; L.ldx = w->ld; L.f32 = f32; L.m = (int)m; L.epi = epilogue; L.scale = scale; L.cap = cap;
-    if (epilogue != EPI_RELU2) {
+    if (!to_act(epilogue)) {
         L.y = dev_y; L.ldy = L.n_store = w->rows;
         return launch_dense(dev, L);
     }
@@ -648,7 +709,7 @@ int candy_hip_dense_matmul(candy_hip_device *dev, const candy_hip_dense *w, cons
 int candy_hip_dense_sweep(candy_hip_device *dev, const candy_hip_dense *const *ws, int n_ws, const float *dev_x, int64_t m,
                           int epilogue, int iters, float *elapsed_ms) {
     CANDY_REQUIRE(dev && ws && n_ws > 0 && dev_x && elapsed_ms && iters > 0 && m > 0 && m <= 1 << 20, "nil argument");
-    CANDY_REQUIRE(epilogue >= EPI_NONE && epilogue <= EPI_CAP, "unknown epilogue %d", epilogue);
+    CANDY_REQUIRE(epilogue >= EPI_NONE && epilogue <= EPI_ACT, "unknown epilogue %d", epilogue);
     for (int i = 0; i < n_ws; ++i)
         CANDY_REQUIRE(ws[i] && ws[i]->dev == dev && ws[i]->rows == ws[0]->rows && ws[i]->cols == ws[0]->cols,
                       "weights of one sweep share a device and a shape");

@@ -1,12 +1,11 @@
-// Layer normalization, alone and chained: a sublayer's result enters the residual sum through a norm of its own and
-// the next sublayer reads a norm of the sum,
-//     x <- x + mult * LN(y) (+ step),   out = LN(x),
-// in one pass over the row.  Everything in f32; `out` is rounded to the activation format on the store.
+// Layer normalization or RMS normalization, alone and chained: a sublayer's result enters the residual sum through a norm
+// of its own and the next sublayer reads a norm of the sum, or the sum itself,
+//     x <- x + mult * N(y) (+ step),   out = N(x) or x,
+// in one pass over the row; y may be spread over partial copies and over the results of routed experts.  Everything in f32; `out` is rounded to the activation format on the store.
 // One workgroup per row, the row in registers; mean and variance in two passes over them.
-// (No counterpart on the reference path this library stands behind, whose norm is RMSNorm, reduce.go:3071-3092.)
+// (The reference path this library stands behind normalizes in front of its sublayers only, reduce.go:3071-3092.)
 #include <algorithm>
 
-#include "blocks.h"
 #include "dense.h"
 
 namespace candy {
@@ -20,20 +19,11 @@ struct NormKernelArgs {
     const int *row_ids;
     int64_t ldx, ldy, ldo;
     size_t y_stride;
-    int y_copies, cols;
+    const float *slots, *slot_weight;
+    int64_t slot_ld;
+    int y_copies, cols, top, rms;
     float mult, eps;
 };
-
-__device__ __forceinline__ float block_sum(float v, float *red) {
-    v = wave_sum(v);
-    const int n_waves = blockDim.x >> 6;
-    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
-    __syncthreads();
-    float t = red[0];
-    for (int w = 1; w < n_waves; ++w) t += red[w];
-    __syncthreads();
-    return t;
-}
 
 // V: float4 per thread; columns past `cols` (inside the padding) hold zeros and stay zero
 template <class AT, int V>
@@ -50,12 +40,15 @@ __global__ __launch_bounds__(256) void k_norm_chain(const NormKernelArgs a) {
 #pragma unroll
         for (int i = 0; i < V; ++i) d[i] = col(i) < padded ? *(const f32x4 *)(p + col(i)) : f32x4{0.f, 0.f, 0.f, 0.f};
     };
-    // in place: d <- (d - mean) * rstd * w + b inside `cols`, 0 outside
+    // in place: d <- (d - mean) * rstd * w + b inside `cols`, 0 outside (RMS: mean and b are 0)
     auto normalize = [&](f32x4 (&d)[V], const float *w, const float *b) {
-        float s = 0.0f;
+        float mean = 0.0f;
+        if (!a.rms) {
+            float s = 0.0f;
 #pragma unroll
-        for (int i = 0; i < V; ++i) s += (d[i][0] + d[i][1]) + (d[i][2] + d[i][3]);
-        const float mean = block_sum(s, red) * inv_n;
+            for (int i = 0; i < V; ++i) s += (d[i][0] + d[i][1]) + (d[i][2] + d[i][3]);
+            mean = block_sum(s, red) * inv_n;
+        }
         float q = 0.0f;
 #pragma unroll
         for (int i = 0; i < V; ++i)
@@ -68,20 +61,29 @@ __global__ __launch_bounds__(256) void k_norm_chain(const NormKernelArgs a) {
 #pragma unroll
         for (int i = 0; i < V; ++i) {
             if (col(i) >= padded) continue;
-            const f32x4 wv = *(const f32x4 *)(w + col(i)), bv = *(const f32x4 *)(b + col(i));  // zero in the padding
+            const f32x4 wv = *(const f32x4 *)(w + col(i));  // zero in the padding, like b
+            const f32x4 bv = b ? *(const f32x4 *)(b + col(i)) : f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
             for (int j = 0; j < 4; ++j) d[i][j] = d[i][j] * rstd * wv[j] + bv[j];
         }
     };
     load_row(a.x + src * a.ldx, x);
-    if (a.y) {
-        const float *yr = a.y + src * a.ldy;
-        load_row(yr, y);
-        for (int c = 1; c < a.y_copies; ++c) {
+    if (a.y || a.slots) {
+#pragma unroll
+        for (int i = 0; i < V; ++i) y[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+        for (int c = 0; a.y && c < a.y_copies; ++c) {
             f32x4 t[V];
-            load_row(yr + (size_t)c * a.y_stride, t);
+            load_row(a.y + src * a.ldy + (size_t)c * a.y_stride, t);
 #pragma unroll
             for (int i = 0; i < V; ++i) y[i] += t[i];
+        }
+        for (int k = 0; a.slots && k < a.top; ++k) {
+            const size_t slot = src * a.top + k;
+            const float g = a.slot_weight[slot];
+            f32x4 t[V];
+            load_row(a.slots + slot * a.slot_ld, t);
+#pragma unroll
+            for (int i = 0; i < V; ++i) y[i] += g * t[i];
         }
         normalize(y, a.post_w, a.post_b);
 #pragma unroll
@@ -98,7 +100,7 @@ __global__ __launch_bounds__(256) void k_norm_chain(const NormKernelArgs a) {
             if (col(i) < padded) *(f32x4 *)(a.x_out + row * a.ldx + col(i)) = x[i];
     }
     if (a.out) {
-        normalize(x, a.pre_w, a.pre_b);
+        if (a.pre_w) normalize(x, a.pre_w, a.pre_b);
         AT *o = (AT *)a.out + row * a.ldo;
         typedef AT at4 __attribute__((ext_vector_type(4)));
 #pragma unroll
@@ -110,7 +112,8 @@ __global__ __launch_bounds__(256) void k_norm_chain(const NormKernelArgs a) {
 int launch_norm_chain(candy_hip_device *dev, const NormArgs &A) {
     CANDY_REQUIRE(A.rows > 0 && A.cols > 0 && A.cols <= 16384, "layer norm takes rows of 1 .. 16384 values, got %d", A.cols);
     NormKernelArgs k{A.x, A.y.p, A.post_w, A.post_b, A.step, A.pre_w, A.pre_b, A.x_out, A.out, A.row_ids,
-                     A.ldx, A.y.ld, A.ldo, A.y.stride, A.y.copies, A.cols, A.mult, A.eps};
+                     A.ldx, A.y.ld, A.ldo, A.y.stride, A.slots, A.slot_weight, A.slot_ld, A.y.copies, A.cols, A.top, A.rms, A.mult,
+                     A.eps};
     const int v = (int)((pad64(A.cols) + 1023) / 1024);
     const dim3 g((unsigned)A.rows), b(256);
 #define CANDY_NORM(AT)                                                                         \
@@ -154,22 +157,24 @@ extern "C" {
 // The kernels work on rows padded to multiples of 64; these two entry points take plain ones and go through the
 // handle's workspace.
 static int norm_op(candy_hip_device *dev, const float *x, const float *y, const float *w, const float *b, float eps,
-                   float mult, const float *step, int64_t rows, int64_t cols, float *out) {
+                   float mult, const float *step, int64_t rows, int64_t cols, float *out, bool rms = false) {
     CANDY_REQUIRE(dev, "device handle is nil");
     CANDY_REQUIRE(rows >= 0 && cols > 0 && cols <= 16384, "layer norm takes rows of 1 .. 16384 values, got %lld", (long long)cols);
     if (rows == 0) return CANDY_HIP_OK;
     CANDY_REQUIRE(rows <= 0x7FFFFFFF / 16384, "too many rows");
-    CANDY_REQUIRE(x && w && b && out, "nil pointer");
+    CANDY_REQUIRE(x && w && (b || rms) && out, "nil pointer");
     if (int rc = use_device(dev)) return rc;
     const int64_t ld = pad64(cols);
     void *ws = nullptr;
     if (int rc = workspace(dev, (size_t)(2 * rows + 3) * ld * sizeof(float), &ws)) return rc;
-    float *px = (float *)ws, *py = px + rows * ld, *pw = py + rows * ld, *pb = pw + ld, *ps = pb + ld;
+    float *px = (float *)ws, *py = px + rows * ld, *pw = py + rows * ld, *pb = pw + ld, *ps = pw + 2 * ld;
     if (int rc = repitch(dev, x, cols, px, ld, rows, cols)) return rc;
     if (int rc = repitch(dev, w, cols, pw, ld, 1, cols)) return rc;
-    if (int rc = repitch(dev, b, cols, pb, ld, 1, cols)) return rc;
+    if (b)
+        if (int rc = repitch(dev, b, cols, pb, ld, 1, cols)) return rc;
+    if (!b) pb = nullptr;
     NormArgs A;
-    A.x = px; A.ldx = ld; A.eps = eps; A.rows = (int)rows; A.cols = (int)cols; A.f32 = true;
+    A.x = px; A.ldx = ld; A.eps = eps; A.rms = rms; A.rows = (int)rows; A.cols = (int)cols; A.f32 = true;
     if (y) {
         if (int rc = repitch(dev, y, cols, py, ld, rows, cols)) return rc;
         A.y.p = py; A.y.ld = (int)ld; A.post_w = pw; A.post_b = pb; A.mult = mult; A.x_out = px;
@@ -193,6 +198,12 @@ int candy_hip_add_layer_norm(candy_hip_device *dev, float *x, const float *y, co
                              float mult, const float *step, int64_t rows, int64_t cols) {
     CANDY_REQUIRE(rows == 0 || y, "nil pointer");
     return norm_op(dev, x, y, w, b, eps, mult, step, rows, cols, x);
+}
+
+int candy_hip_add_rms_norm(candy_hip_device *dev, float *x, const float *y, const float *w, float eps, float mult, int64_t rows,
+                           int64_t cols) {
+    CANDY_REQUIRE(rows == 0 || y, "nil pointer");
+    return norm_op(dev, x, y, w, nullptr, eps, mult, nullptr, rows, cols, x, true);
 }
 
 }  // extern "C"

@@ -49,11 +49,46 @@ class SuvazenConfig(ctypes.Structure):
                 ("norm_eps", c_float), ("residual_mult", c_float), ("logit_scale", c_float), ("logit_softcap", c_float)]
 
 
+class LatentSpec(ctypes.Structure):
+    _fields_ = [("n_heads", c_int32), ("dim", c_int32), ("rot_dim", c_int32), ("vdim", c_int32), ("kv_rank", c_int32),
+                ("q_rank", c_int32), ("scale", c_float), ("rope_base", c_double)]
+
+
+class LruSpec(ctypes.Structure):
+    _fields_ = [("width", c_int32), ("blocks", c_int32), ("taps", c_int32)]
+
+
+class LruParams(ctypes.Structure):
+    _fields_ = [(name, c_void_p) for name in ("by", "bx", "conv", "conv_b", "ra_b", "ri_b", "lam")]
+
+
+class ExpertSpec(ctypes.Structure):
+    _fields_ = [("n_experts", c_int32), ("top", c_int32), ("d_ff", c_int32), ("shared_ff", c_int32)]
+
+
+class ExpertWeights(ctypes.Structure):
+    _fields_ = [(name, c_void_p) for name in ("router", "up", "down", "shared_up", "shared_down")]
+
+
+class GulisunLayer(ctypes.Structure):
+    _fields_ = [("mixer", c_int32), ("kv_from", c_int32), ("has_sink", c_int32), ("reserved", c_int32), ("latent", LatentSpec),
+                ("lru", LruSpec), ("experts", ExpertSpec)]
+
+
+class GulisunConfig(ctypes.Structure):
+    _fields_ = [("n_layers", c_int32), ("d_model", c_int32), ("vocab", c_int32), ("max_pos", c_int32), ("act", c_int32),
+                ("norm_eps", c_float), ("embed_scale", c_float)]
+
+
 ACT_BF16, ACT_F32 = 0, 1
-EPI_NONE, EPI_SQUARED_RELU, EPI_SOFTCAP = 0, 1, 2
+EPI_NONE, EPI_SQUARED_RELU, EPI_SOFTCAP, EPI_ACT = 0, 1, 2, 3
 SV_QK, SV_O, SV_UP, SV_DOWN, SV_HEAD, SV_EMBED = range(6)
 (SV_NORM1, SV_NORM1_BIAS, SV_NORM1B, SV_NORM1B_BIAS, SV_NORM2, SV_NORM2_BIAS, SV_NORM2B, SV_NORM2B_BIAS, SV_SINK, SV_STEP,
  SV_FINAL, SV_FINAL_BIAS) = range(12)
+GL_LATENT, GL_LRU = 0, 1
+(GL_IN, GL_UQ, GL_UKV, GL_UKT, GL_GATES, GL_O, GL_ROUTER, GL_UP, GL_DOWN, GL_SHARED_UP, GL_SHARED_DOWN, GL_EMBED) = range(12)
+(GL_NORM1, GL_NORM2, GL_Q_NORM, GL_KV_NORM, GL_SINK, GL_Y_BIAS, GL_X_BIAS, GL_CONV, GL_CONV_BIAS, GL_RA_BIAS, GL_RI_BIAS, GL_LAM,
+ GL_FINAL) = range(13)
 
 # name -> (restype, argtypes); exactly the symbols include/candy_hip.h declares
 SIGNATURES = {
@@ -136,6 +171,18 @@ SIGNATURES = {
     "candy_hip_layer_norm": (c_int, [c_void_p, c_void_p, c_void_p, c_void_p, c_float, c_int64, c_int64, c_void_p]),
     "candy_hip_add_layer_norm": (c_int, [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_float, c_float, c_void_p,
                                          c_int64, c_int64]),
+    "candy_hip_add_rms_norm": (c_int, [c_void_p, c_void_p, c_void_p, c_void_p, c_float, c_float, c_int64, c_int64]),
+    "candy_hip_pad32": (c_int32, [c_int32]),
+    "candy_hip_pad64": (c_int32, [c_int32]),
+    "candy_hip_latent_row": (c_int32, [POINTER(LatentSpec)]),
+    "candy_hip_latent_attention": (c_int, [c_void_p, POINTER(LatentSpec), c_int, c_void_p, c_void_p, c_void_p, c_float, c_void_p, c_void_p,
+                                           c_void_p, c_int64, c_int32, c_int32, c_void_p, c_int, c_void_p]),
+    "candy_hip_lru_state_floats": (c_int64, [POINTER(LruSpec)]),
+    "candy_hip_lru_gate_rows": (c_int64, [POINTER(LruSpec)]),
+    "candy_hip_lru": (c_int, [c_void_p, POINTER(LruSpec), c_int, c_void_p, POINTER(LruParams), c_void_p, c_void_p, c_int64, c_int32, c_int,
+                              c_void_p]),
+    "candy_hip_experts": (c_int, [c_void_p, POINTER(ExpertSpec), c_int, POINTER(ExpertWeights), c_void_p, c_int64, c_int, c_void_p,
+                                  c_void_p, c_void_p]),
     "candy_hip_attn_row": (c_int, [c_int]),
     "candy_hip_window_attention": (c_int, [c_void_p, POINTER(AttnSpec), c_int, c_void_p, c_int64, c_int32, c_int32, c_void_p,
                                            c_void_p, c_void_p, c_int, c_void_p]),
@@ -154,6 +201,10 @@ SIGNATURES = {
     "candy_hip_suvazen_decoder": (c_void_p, [c_void_p]),
     "candy_hip_suvazen_set_matrix": (c_int, [c_void_p, c_int, c_int, c_void_p]),
     "candy_hip_suvazen_set_vector": (c_int, [c_void_p, c_int, c_int, c_void_p, c_int64]),
+    "candy_hip_gulisun_create": (c_int, [c_void_p, POINTER(GulisunConfig), POINTER(GulisunLayer), POINTER(c_void_p)]),
+    "candy_hip_gulisun_decoder": (c_void_p, [c_void_p]),
+    "candy_hip_gulisun_set_matrix": (c_int, [c_void_p, c_int, c_int, c_void_p]),
+    "candy_hip_gulisun_set_vector": (c_int, [c_void_p, c_int, c_int, c_void_p, c_int64]),
     "candy_hip_qmatmul_sweep": (c_int, [c_void_p, POINTER(c_void_p), c_int, c_void_p, c_int64, c_void_p, c_int, c_int,
                                         POINTER(c_float)]),
     "candy_hip_qmatmul_sustained_sweep": (c_int, [c_void_p, POINTER(c_void_p), c_int, c_int, c_int, c_void_p, c_void_p, c_int,
@@ -599,6 +650,64 @@ class Device:
                                                 v_cache.ptr, ds.ptr if ds else None, int(decode), out.ptr))
         return out.download(np.float32, n * width).reshape(n, width)
 
+    # ---- latent attention, recurrent unit, experts, RMS norm of a result
+    def add_rms_norm(self, x, y, w, eps: float, mult: float) -> np.ndarray:
+        """x + mult * rms_norm(y)"""
+        x = np.ascontiguousarray(x, np.float32)
+        cols = x.shape[-1]
+        dx, dy, dw = self._f32(x), self._f32(y), self._f32(w)
+        _check(lib().candy_hip_add_rms_norm(self.handle, dx.ptr, dy.ptr, dw.ptr, eps, mult, x.size // cols, cols))
+        return dx.download(np.float32, x.size).reshape(x.shape)
+
+    def latent_attention(self, spec: LatentSpec, act: int, q, dkv, kv_norm, eps: float, ukv: Dense, ukt: Dense, pos0: int, max_pos: int,
+                         cache: "Buffer", sink=None, decode: bool = False) -> np.ndarray:
+        """Rows at positions pos0 .. in the padded layouts of include/candy_hip.h; dkv None: the cache holds them already."""
+        q = np.ascontiguousarray(q, np.float32)
+        n, width = q.shape[0], spec.n_heads * lib().candy_hip_pad32(spec.vdim)
+        row = lib().candy_hip_latent_row(byref(spec))
+        dk = lib().candy_hip_pad32(spec.dim) + lib().candy_hip_pad32(spec.rot_dim)
+        if q.shape[1] != spec.n_heads * dk or (dkv is not None and np.shape(dkv) != (n, row)):
+            raise ValueError("rows do not fit the spec")
+        if cache.nbytes < max_pos * row * (4 if act == ACT_F32 else 2):
+            raise ValueError("cache too small")
+        dq, out = self._f32(q), self.alloc(n * width * 4)
+        dd = self._f32(dkv) if dkv is not None else None
+        dn = self._f32(kv_norm) if dkv is not None else None
+        ds = self._f32(sink) if sink is not None else None
+        _check(lib().candy_hip_latent_attention(self.handle, byref(spec), act, dq.ptr, dd.ptr if dd else None, dn.ptr if dn else None, eps,
+                                                ukv.handle, ukt.handle, ds.ptr if ds else None, n, pos0, max_pos, cache.ptr, int(decode),
+                                                out.ptr))
+        return out.download(np.float32, n * width).reshape(n, width)
+
+    def lru(self, spec: LruSpec, act: int, z, params: dict, gates: Dense, state: "Buffer", pos0: int, decode: bool = False) -> np.ndarray:
+        """z [n, 2 * pad64(width)]; params: the fields of LruParams, padded."""
+        z = np.ascontiguousarray(z, np.float32)
+        n, wp = z.shape[0], lib().candy_hip_pad64(spec.width)
+        if z.shape[1] != 2 * wp or state.nbytes < 4 * lib().candy_hip_lru_state_floats(byref(spec)):
+            raise ValueError("rows or state do not fit the spec")
+        bufs = {k: self._f32(np.ascontiguousarray(v, np.float32)) for k, v in params.items()}
+        for k, b in bufs.items():
+            if b.nbytes < 4 * wp * (spec.taps if k == "conv" else 1):
+                raise ValueError(f"{k} is not padded")
+        p = LruParams(**{k: b.ptr for k, b in bufs.items()})
+        dz, out = self._f32(z), self.alloc(n * spec.width * 4)
+        _check(lib().candy_hip_lru(self.handle, byref(spec), act, dz.ptr, byref(p), gates.handle, state.ptr, n, pos0, int(decode), out.ptr))
+        return out.download(np.float32, n * spec.width).reshape(n, spec.width)
+
+    def experts(self, spec: ExpertSpec, act: int, weights: dict, x, decode: bool = False):
+        """weights: the fields of ExpertWeights as Dense; returns the result, and for several rows the choice and its weights."""
+        x = np.ascontiguousarray(x, np.float32)
+        n, d = x.shape
+        w = ExpertWeights(**{k: v.handle for k, v in weights.items()})
+        dx, out = self._f32(x), self.alloc(n * d * 4)
+        ids, wts = (None, None) if decode else (self.alloc(n * spec.top * 4), self.alloc(n * spec.top * 4))
+        _check(lib().candy_hip_experts(self.handle, byref(spec), act, byref(w), dx.ptr, n, int(decode), out.ptr,
+                                       ids.ptr if ids else None, wts.ptr if wts else None))
+        y = out.download(np.float32, n * d).reshape(n, d)
+        if decode:
+            return y
+        return y, ids.download(np.int32, n * spec.top).reshape(n, -1), wts.download(np.float32, n * spec.top).reshape(n, -1)
+
     # ---- timing
     def qmatmul_sweep(self, weights: list, x_buf: "Buffer", m: int, y_buf: "Buffer", iters: int,
                       quantize_each: bool = True) -> float:
@@ -774,23 +883,40 @@ class Llama(Decoder):
         _check(lib().candy_hip_llama_set_kv_f16(self.model, int(enable)))
 
 
-class Suvazen(Decoder):
-    """Suvazen decoder on the device (candy_amd/suvazen.py builds one from a model folder)."""
+class _LayerModel(Decoder):
+    """A decoder created from a configuration and a list of layers (weights stay owned by the caller, vectors are copied)."""
 
-    def __init__(self, dev: Device, cfg: SuvazenConfig, layers: list):
+    NAME, LAYER = "", None
+
+    def __init__(self, dev: Device, cfg, layers: list):
         self.dev, self.cfg = dev, cfg
-        self.layers = (SuvazenLayer * len(layers))(*layers)
+        self.layers = (self.LAYER * len(layers))(*layers)
         h = c_void_p()
-        _check(lib().candy_hip_suvazen_create(dev.handle, byref(cfg), self.layers, byref(h)))
+        _check(self._call("create")(dev.handle, byref(cfg), self.layers, byref(h)))
         self.model = h.value
-        self.handle = lib().candy_hip_suvazen_decoder(self.model)
+        self.handle = self._call("decoder")(self.model)
         self.width, self.vocab, self.max_pos = cfg.d_model, cfg.vocab, cfg.max_pos
         self._keep = []
 
+    def _call(self, what: str):
+        return getattr(lib(), f"candy_hip_{self.NAME}_{what}")
+
     def set_matrix(self, which: int, layer: int, w: Dense):
         self._keep.append(w)
-        _check(lib().candy_hip_suvazen_set_matrix(self.model, which, layer, w.handle))
+        _check(self._call("set_matrix")(self.model, which, layer, w.handle))
 
     def set_vector(self, which: int, layer: int, values: np.ndarray):
         v = np.ascontiguousarray(values, np.float32).reshape(-1)
-        _check(lib().candy_hip_suvazen_set_vector(self.model, which, layer, v.ctypes.data, v.size))
+        _check(self._call("set_vector")(self.model, which, layer, v.ctypes.data, v.size))
+
+
+class Suvazen(_LayerModel):
+    """Suvazen decoder on the device (candy_amd/suvazen.py builds one from a model folder)."""
+
+    NAME, LAYER = "suvazen", SuvazenLayer
+
+
+class Gulisun(_LayerModel):
+    """Gulisun decoder on the device (candy_amd/gulisun.py builds one from a model folder)."""
+
+    NAME, LAYER = "gulisun", GulisunLayer

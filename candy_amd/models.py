@@ -7,7 +7,7 @@ from __future__ import annotations
 import json
 import os
 
-from . import gguf, hip, suvazen
+from . import gguf, gulisun, hip, suvazen
 
 DEFAULT_MAX_POS = 4096
 
@@ -25,6 +25,7 @@ def _llama(dev, path, max_pos, act):
 # architecture -> loader(dev, path, max_pos or None, activation format) -> hip.Decoder
 ARCHITECTURES = {
     "llama": _llama,
+    "Gulisun": lambda dev, path, max_pos, act: gulisun.load(dev, path, max_pos or DEFAULT_MAX_POS, act),
     "Suvazen": lambda dev, path, max_pos, act: suvazen.load(dev, path, max_pos or DEFAULT_MAX_POS, act),
 }
 

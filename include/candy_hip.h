@@ -376,10 +376,12 @@ int candy_hip_dense_info(const candy_hip_dense *w, int64_t *rows, int64_t *cols,
  * widened exactly. */
 enum candy_hip_act { CANDY_HIP_ACT_BF16 = 0, CANDY_HIP_ACT_F32 = 1 };
 /* What follows the contraction z: NONE z; SQUARED_RELU max(z, 0)^2; SOFTCAP cap * tanh(scale * z / cap), or scale * z
- * with cap 0. */
-enum candy_hip_epilogue { CANDY_HIP_EPI_NONE = 0, CANDY_HIP_EPI_SQUARED_RELU = 1, CANDY_HIP_EPI_SOFTCAP = 2 };
+ * with cap 0; ACT z in the activation format. */
+enum candy_hip_epilogue {
+    CANDY_HIP_EPI_NONE = 0, CANDY_HIP_EPI_SQUARED_RELU = 1, CANDY_HIP_EPI_SOFTCAP = 2, CANDY_HIP_EPI_ACT = 3
+};
 /* y[m, rows] = epilogue(x[m, cols] . W^T), f32 in and out (x is converted on the device where act asks for it; the
- * squared ReLU's output is rounded to the activation format, as the next contraction reads it). */
+ * output of SQUARED_RELU and ACT is rounded to the activation format, as the next contraction reads it). */
 int candy_hip_dense_matmul(candy_hip_device *dev, const candy_hip_dense *w, const float *dev_x, int64_t m, int act,
                            int epilogue, float scale, float cap, float *dev_y);
 /* `iters` bfloat16 contractions back to back over n_ws weights of one shape (activations already bfloat16), timed with
@@ -393,6 +395,9 @@ int candy_hip_layer_norm(candy_hip_device *dev, const float *x, const float *w, 
  * entering the residual sum through a norm of its own. */
 int candy_hip_add_layer_norm(candy_hip_device *dev, float *x, const float *y, const float *w, const float *b, float eps,
                              float mult, const float *step, int64_t rows, int64_t cols);
+/* The same with an RMS norm: x += mult * y / sqrt(mean(y^2) + eps) * w. */
+int candy_hip_add_rms_norm(candy_hip_device *dev, float *x, const float *y, const float *w, float eps, float mult, int64_t rows,
+                           int64_t cols);
 
 /* One attention layer: grouped heads, rotary positions on the first rope_dims dimensions of a head (pairs i,
  * i + rope_dims/2; angle p * rope_base^(-2i/rope_dims)), values = the keys before rotation, scores
@@ -416,6 +421,67 @@ int candy_hip_attn_row(int head_dim);   /* values per position and head in the c
 int candy_hip_window_attention(candy_hip_device *dev, const candy_hip_attn_spec *spec, int act, const float *qk, int64_t n,
                                int32_t pos0, int32_t max_pos, void *k_cache, void *v_cache, const float *sink, int decode,
                                float *out);
+
+/* Latent attention: a layer caches one row per position, shared by its heads - a normed latent c of kv_rank values and a
+ * rotated key part of rot_dim values.  Head h scores position j with
+ *     scale * ((Wuk_h c_j) . q_h[0 .. dim) + kr_j . rot(q_h[dim .. dim + rot_dim)))
+ * over all j up to its own position, its value there is Wuv_h c_j [vdim], and the softmax denominator may also hold
+ * exp(sink_h).  Rotation turns all rot_dim dimensions (pairs i, i + rot_dim/2; angle p * rope_base^(-2i/rot_dim)).
+ * Prompts expand keys and values of every head; a decode step contracts q_h with Wuk_h and works on the cached rows.
+ * Device layouts pad with zeros: dim, rot_dim and vdim to multiples of 32 (candy_hip_pad32), ranks to multiples of 64. */
+typedef struct candy_hip_latent_spec {
+    int32_t n_heads, dim, rot_dim, vdim, kv_rank, q_rank;
+    float scale;
+    double rope_base;
+} candy_hip_latent_spec;
+int32_t candy_hip_pad32(int32_t n);
+int32_t candy_hip_pad64(int32_t n);
+/* Values per position in the cache: pad64(kv_rank) + pad32(rot_dim); 0 for a spec the kernels do not take. */
+int32_t candy_hip_latent_row(const candy_hip_latent_spec *spec);
+/* The mechanism between its projections, for n tokens at positions pos0 ..: q [n, n_heads * (pad32(dim) + pad32(rot_dim))]
+ * f32 before rotation; dkv [n, pad64(kv_rank) + pad32(rot_dim)] f32 before norm and rotation, or NULL when the cache
+ * holds the rows already (a layer that shares another's); kv_norm [kv_rank] with dkv; cache [max_pos, latent_row] of the
+ * activation format; ukv [n_heads * (pad32(dim) + pad32(vdim)), kv_rank]: every head's Wuk, then every head's Wuv; ukt
+ * [n_heads * pad64(kv_rank), dim]: every head's Wuk transposed; out [n, n_heads * pad32(vdim)] f32.
+ * decode != 0 (n = 1): the kernels of the decode step. */
+int candy_hip_latent_attention(candy_hip_device *dev, const candy_hip_latent_spec *spec, int act, const float *q, const float *dkv,
+                               const float *kv_norm, float eps, const candy_hip_dense *ukv, const candy_hip_dense *ukt,
+                               const float *sink, int64_t n, int32_t pos0, int32_t max_pos, void *cache, int decode, float *out);
+
+/* Real-gated linear recurrent unit behind its projections: y = gelu_tanh(zy + by), v = zx + bx, u = the causal
+ * convolution of v per channel (taps columns, the last the current token's) + bias; with u cut into `blocks` equal parts,
+ * r = sigmoid(A_b u_b + .), i = sigmoid(I_b u_b + .), a = exp(-8 r softplus(lam)), S = a S + sqrt(1 - a^2) i u; the result
+ * is S * y.  State per sequence: S and the last taps - 1 values of v, both f32; at position 0 both are zero. */
+typedef struct candy_hip_lru_spec {
+    int32_t width, blocks, taps;
+} candy_hip_lru_spec;
+/* Vectors of one unit, each a device array: by, bx, conv_b, lam, ra_b, ri_b [pad64(width)]; conv [taps, pad64(width)]. */
+typedef struct candy_hip_lru_params {
+    const float *by, *bx, *conv, *conv_b, *ra_b, *ri_b, *lam;
+} candy_hip_lru_params;
+/* Floats of the state; rows of the gate matrix: with s = pad64(width / blocks), every block has s / 64 groups of 64 rows
+ * of A_b followed by the same 64 rows of I_b (zero rows past the block's size), columns width / blocks. */
+int64_t candy_hip_lru_state_floats(const candy_hip_lru_spec *spec);
+int64_t candy_hip_lru_gate_rows(const candy_hip_lru_spec *spec);
+/* z [n, 2 * pad64(width)] f32: zy, then zx; state: device memory, carried; out [n, width] f32. */
+int candy_hip_lru(candy_hip_device *dev, const candy_hip_lru_spec *spec, int act, const float *z, const candy_hip_lru_params *params,
+                  const candy_hip_dense *gates, float *state, int64_t n, int32_t pos0, int decode, float *out);
+
+/* Routed experts with squared-ReLU feed-forwards: scores = softmax(router . x) in f32, the `top` largest chosen (lower
+ * number first among equals), weights = their scores over their sum (+ 1e-20); the result is the weighted sum of the
+ * chosen experts' down . max(up . x, 0)^2, plus that of a shared one for every token (shared_ff 0: none). */
+typedef struct candy_hip_expert_spec {
+    int32_t n_experts, top, d_ff, shared_ff;
+} candy_hip_expert_spec;
+/* Matrices: router [n_experts, d]; up [n_experts * pad64(d_ff), d], down [n_experts * pad64(d), d_ff], an expert's rows
+ * padded with zeros; shared_up [shared_ff, d], shared_down [d, shared_ff] or NULL. */
+typedef struct candy_hip_expert_weights {
+    const candy_hip_dense *router, *up, *down, *shared_up, *shared_down;
+} candy_hip_expert_weights;
+/* x [n, d] f32 -> out [n, d] f32; ids / weights (optional, [n, top]) receive the choice, largest score first.
+ * decode != 0 (n = 1): the kernels of the decode step. */
+int candy_hip_experts(candy_hip_device *dev, const candy_hip_expert_spec *spec, int act, const candy_hip_expert_weights *w,
+                      const float *x, int64_t n, int decode, float *out, int32_t *ids, float *weights);
 
 /* ------------------------------------------------------------------ any decoder
  * What candy_hip_llama_decode and its neighbours do, for every model of the library. */
@@ -479,6 +545,58 @@ candy_hip_decoder *candy_hip_suvazen_decoder(candy_hip_suvazen *m);   /* free th
 /* Matrices are borrowed and must outlive the model. */
 int candy_hip_suvazen_set_matrix(candy_hip_suvazen *m, int which, int layer, const candy_hip_dense *w);
 int candy_hip_suvazen_set_vector(candy_hip_suvazen *m, int which, int layer, const float *host, int64_t count);
+
+/* ------------------------------------------------------------------ Gulisun decoder
+ * x = scale * embed[token]; every layer x += norm1(mixer(x)), then x += norm2(experts(x)), RMS norms with weight on the
+ * results only; mixer: latent attention (of its own, or over another layer's cache) or the recurrent unit above, between
+ * its projections; the experts are absent with n_experts 0.  logits = embed . final_norm(x).
+ * A decoder with a recurrent layer takes positions in order: 0, or the one behind the last token it was fed. */
+typedef struct candy_hip_gulisun candy_hip_gulisun;
+enum candy_hip_gulisun_mixer { CANDY_HIP_GL_LATENT = 0, CANDY_HIP_GL_LRU = 1 };
+typedef struct candy_hip_gulisun_layer {
+    int32_t mixer;             /* enum candy_hip_gulisun_mixer                                           */
+    int32_t kv_from;           /* LATENT: the earlier layer whose cache this one reads, or -1: its own   */
+    int32_t has_sink;
+    int32_t reserved;
+    candy_hip_latent_spec latent;
+    candy_hip_lru_spec lru;
+    candy_hip_expert_spec experts;
+} candy_hip_gulisun_layer;
+typedef struct candy_hip_gulisun_config {
+    int32_t n_layers, d_model, vocab, max_pos;
+    int32_t act;               /* enum candy_hip_act */
+    float norm_eps, embed_scale;
+} candy_hip_gulisun_config;
+
+enum candy_hip_gulisun_matrix {   /* bfloat16; padded as the mechanisms above say */
+    CANDY_HIP_GL_IN = 0,       /* LATENT: Wdq [pad64(q_rank) rows], then (own cache) Wdkv [pad64(kv_rank) + pad32(rot_dim) rows];
+                                  LRU: Wy, Wx [pad64(width) rows each]; columns d_model                  */
+    CANDY_HIP_GL_UQ = 1,       /* [n_heads * (pad32(dim) + pad32(rot_dim)), q_rank]                      */
+    CANDY_HIP_GL_UKV = 2,
+    CANDY_HIP_GL_UKT = 3,
+    CANDY_HIP_GL_GATES = 4,
+    CANDY_HIP_GL_O = 5,        /* [d_model, n_heads * pad32(vdim)] or [d_model, width]                   */
+    CANDY_HIP_GL_ROUTER = 6,
+    CANDY_HIP_GL_UP = 7,
+    CANDY_HIP_GL_DOWN = 8,
+    CANDY_HIP_GL_SHARED_UP = 9,
+    CANDY_HIP_GL_SHARED_DOWN = 10,
+    CANDY_HIP_GL_EMBED = 11    /* [vocab, d_model], layer = -1                                           */
+};
+enum candy_hip_gulisun_vector {   /* f32, copied */
+    CANDY_HIP_GL_NORM1 = 0, CANDY_HIP_GL_NORM2 = 1,                        /* [d_model]      */
+    CANDY_HIP_GL_Q_NORM = 2, CANDY_HIP_GL_KV_NORM = 3, CANDY_HIP_GL_SINK = 4,
+    CANDY_HIP_GL_Y_BIAS = 5, CANDY_HIP_GL_X_BIAS = 6,                      /* [width]        */
+    CANDY_HIP_GL_CONV = 7,                                                 /* [taps * width], tap by tap */
+    CANDY_HIP_GL_CONV_BIAS = 8, CANDY_HIP_GL_RA_BIAS = 9, CANDY_HIP_GL_RI_BIAS = 10, CANDY_HIP_GL_LAM = 11,
+    CANDY_HIP_GL_FINAL = 12                                                /* layer = -1     */
+};
+int candy_hip_gulisun_create(candy_hip_device *dev, const candy_hip_gulisun_config *cfg,
+                             const candy_hip_gulisun_layer *layers, candy_hip_gulisun **out);
+candy_hip_decoder *candy_hip_gulisun_decoder(candy_hip_gulisun *m);   /* free through the decoder */
+/* Matrices are borrowed and must outlive the model. */
+int candy_hip_gulisun_set_matrix(candy_hip_gulisun *m, int which, int layer, const candy_hip_dense *w);
+int candy_hip_gulisun_set_vector(candy_hip_gulisun *m, int which, int layer, const float *host, int64_t count);
 
 /* ------------------------------------------------------------------ timing (HIP events on the handle's stream) */
 /* Runs `iters` contractions back to back, iteration i using weight ws[i % n_ws] (all the same
