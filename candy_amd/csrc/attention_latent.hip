@@ -529,7 +529,7 @@ __global__ __launch_bounds__(256) void k_latent_merge(const LatentArgs a, const 
     for (int it = 0; it < 2; ++it)
 #pragma unroll
         for (int s = 0; s < AHEAD; ++s) wf[it][s] = *(const u32x4v *)(w + (size_t)it * 4 * ldw + min(s * 128 + l16 * 8, ldw - 8));
-    const int pitch = a.kv_p + 4, C4 = a.kv_p >> 2, SG = max(256 / C4, 1);
+    const int pitch = a.kv_p + 4, C4 = a.kv_p >> 2, SG = 256 / C4;   // kv_p is at most 1024
     const float *p = part + (size_t)h * n_splits * pitch;
     float ms = LOW, ls = 0.0f;
     if (lane < n_splits) {
@@ -542,23 +542,17 @@ __global__ __launch_bounds__(256) void k_latent_merge(const LatentArgs a, const 
     const float f = e / (wave_sum(ls * e) + (a.sink ? __builtin_amdgcn_exp2f(sink - m) : 0.0f));
     if (wave == 0) factor[lane] = f;
     __syncthreads();
-    const int sg = tid / C4;
-    for (int c4 = tid % C4; c4 < C4; c4 += 256) {   // more than one round only for C4 > 256, where SG is 1
-        f32x4 o{0.f, 0.f, 0.f, 0.f};
-        if (sg < SG)
-            for (int s = sg; s < n_splits; s += SG) o += *(const f32x4 *)(p + (size_t)s * pitch + 4 * c4) * factor[s];
-        if (SG == 1) *(f32x4 *)(lat + 4 * c4) = o;
-        else red[tid] = o;
+    const int sg = tid / C4, c4 = tid % C4;   // thread: splits sg, sg + SG, ... of four columns
+    f32x4 o{0.f, 0.f, 0.f, 0.f};
+    if (sg < SG)
+        for (int s = sg; s < n_splits; s += SG) o += *(const f32x4 *)(p + (size_t)s * pitch + 4 * c4) * factor[s];
+    red[tid] = o;
+    __syncthreads();
+    if (tid < C4) {
+        for (int s = 1; s < SG; ++s) o += red[s * C4 + tid];
+        *(f32x4 *)(lat + 4 * tid) = o;
     }
     __syncthreads();
-    if (SG > 1) {
-        for (int c4 = tid; c4 < C4; c4 += 256) {
-            f32x4 o = red[c4];
-            for (int s = 1; s < SG; ++s) o += red[s * C4 + c4];
-            *(f32x4 *)(lat + 4 * c4) = o;
-        }
-        __syncthreads();
-    }
     float acc[2] = {0.f, 0.f};
     for (int k0 = 0; k0 < ldw; k0 += 128) {
         const int k = k0 + l16 * 8;

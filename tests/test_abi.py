@@ -73,8 +73,9 @@ def test_nil_and_shape_errors_do_not_need_a_device():
     assert b"unknown quantized format" in L.candy_hip_last_error()
     assert L.candy_hip_matmul_f32(None, None, None, None, 1, 0, 1, 1, 0) == 1
     assert b"invalid matrix dimensions" in L.candy_hip_last_error()  # cpu/storage.go:877-879
-    # the other decoder and the generic entry points
+    # the other decoders and the generic entry points
     assert L.candy_hip_suvazen_create(None, None, None, ctypes.byref(out)) == 1
+    assert L.candy_hip_gulisun_create(None, None, None, ctypes.byref(out)) == 1
     assert L.candy_hip_decoder_decode(None, 0, 0, None, None) == 1
     assert L.candy_hip_decoder_prefill_rows(None, None, 1, 0, None, 0, None) == 1
     assert L.candy_hip_decoder_free(None) == 0
