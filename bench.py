@@ -410,6 +410,35 @@ def build_llama_like(dev, size, max_pos, seed=8100):
     return model, nbytes + synth.weight_nbytes(synth.Q6_K, c["vocab"], d), macs
 
 
+def decoder_rows(dev, tag, model, vocab, prompts, n_decode, weight_bytes, kv_bytes, macs):
+    """Prefill and greedy decode behind it, per prompt length.  kv_bytes(seen): cache and state a step reads; macs: per
+    token, in the layers' projections."""
+    rows = []
+    for n in prompts:
+        prompt = [int(t) for t in np.random.default_rng(n).integers(0, vocab, n)]
+        for _ in range(6):
+            tok, _ = model.prefill(prompt, 0, want_logits=False)
+        dev.synchronize()
+        reps = 5
+        t0 = time.perf_counter()
+        for _ in range(reps):
+            tok, _ = model.prefill(prompt, 0, want_logits=False)
+        dev.synchronize()
+        pre = (time.perf_counter() - t0) / reps
+        chosen = model.generate(tok, n, 4)
+        t0 = time.perf_counter()
+        model.generate(chosen[-1], n + 4, n_decode)
+        dev.synchronize()
+        dec = (time.perf_counter() - t0) / n_decode
+        bpt = weight_bytes + kv_bytes(n + 4 + n_decode // 2)
+        rows.append({"prompt": n, "prefill_ms": round(pre * 1e3, 3), "prefill_tok_s": round(n / pre, 1),
+                     "prefill_linear_TFLOPs": round(2.0 * macs * n / pre / 1e12, 1),
+                     "decode_ms_per_token": round(dec * 1e3, 4), "decode_tok_s": round(1 / dec, 2),
+                     "decode_bytes_per_token": bpt, "decode_hbm_frac": round(bpt / dec / 1e9 / HBM_PEAK_GBPS, 4)})
+        log(f"  {tag}: {rows[-1]}")
+    return rows
+
+
 def suvazen_leg(dev, sizes, prompts=(512, 2048), n_decode=64, models=("suvazen", "llama"), eager=False):
     """Prefill and decode of the Suvazen decoder beside the Llama decoder at equal layer shapes."""
     out = {}
@@ -418,40 +447,110 @@ def suvazen_leg(dev, sizes, prompts=(512, 2048), n_decode=64, models=("suvazen",
         window = 1536
         for which in models:
             log(f"building {which} {name} ...")
-            max_pos = max(prompts) + n_decode + 8
+            max_pos = max(prompts) + n_decode + 16
             if which == "suvazen":
                 model, wbytes, macs = build_suvazen(dev, size, max_pos, window)
             else:
                 model, wbytes, macs = build_llama_like(dev, size, max_pos)
             if eager:
                 model.set_graph(False)
-            rows = []
-            for n in prompts:
-                prompt = [int(t) for t in np.random.default_rng(n).integers(0, size["vocab"], n)]
-                for _ in range(6):
-                    tok, _ = model.prefill(prompt, 0, want_logits=False)
-                dev.synchronize()
-                reps = 5
-                t0 = time.perf_counter()
-                for _ in range(reps):
-                    tok, _ = model.prefill(prompt, 0, want_logits=False)
-                dev.synchronize()
-                pre = (time.perf_counter() - t0) / reps
-                model.generate(tok, n, 4)
-                t0 = time.perf_counter()
-                model.generate(tok, n, n_decode)
-                dev.synchronize()
-                dec = (time.perf_counter() - t0) / n_decode
-                # the Llama decoder's cache is f32, Suvazen's bfloat16 and read within the window only
-                seen = n + n_decode // 2
-                kv = 2 * size["n_layers"] * size["n_kv_heads"] * size["head_dim"] * (min(seen, window) * 2 if which == "suvazen" else seen * 4)
-                bpt = wbytes + kv
-                rows.append({"prompt": n, "prefill_ms": round(pre * 1e3, 3), "prefill_tok_s": round(n / pre, 1),
-                             "prefill_linear_TFLOPs": round(2.0 * macs * n / pre / 1e12, 1),
-                             "decode_ms_per_token": round(dec * 1e3, 4), "decode_tok_s": round(1 / dec, 2),
-                             "decode_bytes_per_token": bpt, "decode_hbm_frac": round(bpt / dec / 1e9 / HBM_PEAK_GBPS, 4)})
-                log(f"  {which} {name}: {rows[-1]}")
-            res[which] = rows
+            # the Llama decoder's cache is f32, Suvazen's bfloat16 and read within the window only
+            per_pos = 2 * size["n_layers"] * size["n_kv_heads"] * size["head_dim"]
+            kv = (lambda seen: per_pos * min(seen, window) * 2) if which == "suvazen" else (lambda seen: per_pos * seen * 4)
+            res[which] = decoder_rows(dev, f"{which} {name}", model, size["vocab"], prompts, n_decode, wbytes, kv, macs)
+            model.free()
+        out[name] = res
+    return out
+
+
+# ------------------------------------------------------------------ --gulisun
+# Layer shapes in the manner of published models; `plain`: the Suvazen decoder's layers of the same width, depth and
+# active feed-forward width beside them.
+GULISUN_SIZES = {
+    # many small experts
+    "fine": dict(n_layers=16, width=2048, vocab=102400, heads=16, dim=128, rot_dim=64, vdim=128, kv_rank=512, q_rank=1024,
+                 lru=2560, blocks=10, taps=4, experts=64, top=6, ff=1408, shared=2816,
+                 plain=dict(n_layers=16, d_model=2048, n_heads=16, n_kv_heads=8, head_dim=128, d_ffn=11264, vocab=102400)),
+    # few large ones
+    "coarse": dict(n_layers=16, width=4096, vocab=128256, heads=32, dim=128, rot_dim=64, vdim=128, kv_rank=512, q_rank=1536,
+                   lru=4096, blocks=16, taps=4, experts=16, top=4, ff=2048, shared=6144,
+                   plain=dict(n_layers=16, d_model=4096, n_heads=32, n_kv_heads=8, head_dim=128, d_ffn=14336, vocab=128256)),
+}
+
+
+def build_gulisun(dev, c, max_pos, seed=700):
+    """Random-init Gulisun: of four layers, the first has a cache of its own, the second is recurrent, the third reads the
+    first's cache, the fourth has its own and no sink.  One draw per matrix shape (every layer and expert has a device
+    copy of its own).  Returns (model, weight bytes of a decode step, function of positions -> cache and state bytes of a
+    step, multiply-adds per token in the layers)."""
+    from candy_amd import gulisun, hip
+    d, H = c["width"], c["heads"]
+    dk = c["dim"] + c["rot_dim"]
+    mlp = {"kind": "moe", "router": {"experts": c["experts"], "top": c["top"]}, "expert": {"ff": c["ff"]}, "shared": {"ff": c["shared"]}}
+    layers = []
+    for i in range(c["n_layers"]):
+        mixer = {"heads": H, "dim": c["dim"], "rot_dim": c["rot_dim"], "vdim": c["vdim"], "kv_rank": c["kv_rank"], "q_rank": c["q_rank"],
+                 "scale": dk ** -0.5, "rot": {"base": 500000.0, "dims": c["rot_dim"]}}
+        kind = ("latent_attention", "rglru", "latent_attention", "latent_attention_2")[i % 4]
+        if kind == "rglru":
+            mixer = {"width": c["lru"], "blocks": c["blocks"], "conv": c["taps"]}
+        elif i % 4 == 2:
+            mixer["kv_from"] = i - 2
+        layers.append({"type": kind, "mixer": mixer, "mlp": mlp})
+    cfg = {"vocab": c["vocab"], "width": d, "norm": {"eps": 1e-5}, "embedding": {"scale": 45.0}, "layers": layers}
+    size, rng, draws = c["lru"] // c["blocks"], np.random.Generator(np.random.Philox(seed)), {}
+    shapes = {"embed": (c["vocab"], d), "dq": (c["q_rank"], d), "uq": (H * dk, c["q_rank"]), "dkv": (c["kv_rank"] + c["rot_dim"], d),
+              "uk": (H * c["dim"], c["kv_rank"]), "uv": (H * c["vdim"], c["kv_rank"]), "y": (c["lru"], d), "x": (c["lru"], d),
+              "ra": (c["blocks"], size, size), "ri": (c["blocks"], size, size), "router": (c["experts"], d)}
+    vectors = {"norm1": d, "norm2": d, "final.norm": d, "dq.norm": c["q_rank"], "dkv.norm": c["kv_rank"], "sink": H, "y.b": c["lru"],
+               "x.b": c["lru"], "conv": (c["lru"], c["taps"]), "conv.b": c["lru"], "ra.b": c["lru"], "ri.b": c["lru"], "lam": c["lru"]}
+
+    class Tensors:
+        def bits(self, name):
+            kind = name.split(".", 2)[-1] if name.startswith("l") else name
+            shape = shapes.get(kind)
+            if kind == "o":
+                shape = (d, c["lru"] if layers[int(name[1:].split(".")[0])]["type"] == "rglru" else H * c["vdim"])
+            elif shape is None:
+                ff = c["shared"] if kind.startswith("shared") else c["ff"]
+                shape = (ff, d) if kind.endswith("up") else (d, ff)
+            if shape not in draws:
+                draws[shape] = hip.bf16_bits(rng.standard_normal(shape, dtype=np.float32) * np.float32(0.02))
+            return draws[shape]
+
+        def f32(self, name):
+            kind = name.split(".", 2)[-1] if name.startswith("l") and ".mix." in name else name.split(".", 1)[-1] if name.startswith("l") else name
+            return np.ones(vectors[kind], np.float32) if "norm" in kind else np.full(vectors[kind], -0.5, np.float32)
+
+    model = gulisun.build(dev, cfg, Tensors(), max_pos)
+    q, ukv, o = H * dk * c["q_rank"], H * (c["dim"] + c["vdim"]) * c["kv_rank"], d * H * c["vdim"]
+    n_lru = c["n_layers"] // 4
+    own, reads = 2 * n_lru, 3 * n_lru
+    down = d * (c["q_rank"] * reads + (c["kv_rank"] + c["rot_dim"]) * own)
+    macs = down + reads * (q + ukv + o) + n_lru * c["lru"] * (3 * d + 2 * size)
+    macs += c["n_layers"] * d * (c["experts"] + 2 * (c["top"] * c["ff"] + c["shared"]))
+    row = 2 * (c["kv_rank"] + c["rot_dim"])
+    state = 4 * c["lru"] * (1 + c["taps"]) * n_lru
+    return model, 2 * (macs + c["vocab"] * d), lambda seen: reads * row * seen + state, macs
+
+
+def gulisun_leg(dev, sizes, prompts=(512, 2048), n_decode=64, models=("gulisun", "suvazen"), eager=False):
+    """Prefill and decode of the Gulisun decoder beside the Suvazen decoder at equal width, depth and active feed-forward."""
+    out = {}
+    for name in sizes:
+        c, res = GULISUN_SIZES[name], {}
+        plain = c["plain"]
+        for which in models:
+            log(f"building {which} {name} ...")
+            max_pos = max(prompts) + n_decode + 16
+            if which == "gulisun":
+                model, wbytes, kv, macs = build_gulisun(dev, c, max_pos)
+            else:
+                model, wbytes, macs = build_suvazen(dev, plain, max_pos, window=max_pos)
+                kv = lambda seen: 4 * plain["n_layers"] * plain["n_kv_heads"] * plain["head_dim"] * seen  # noqa: E731
+            if eager:
+                model.set_graph(False)
+            res[which] = decoder_rows(dev, f"{which} {name}", model, c["vocab"], prompts, n_decode, wbytes, kv, macs)
             model.free()
         out[name] = res
     return out
@@ -542,6 +641,10 @@ def main():
                     help="instead of the default workload: prefill and decode of the Suvazen decoder beside the Llama decoder at "
                          "equal layer shapes (sizes: 8b, 1b)")
     ap.add_argument("--suvazen-models", default="suvazen,llama", help="which decoders --suvazen runs")
+    ap.add_argument("--gulisun", nargs="?", const="fine,coarse", metavar="SIZES",
+                    help="instead of the default workload: prefill and decode of the Gulisun decoder beside the Suvazen decoder at "
+                         "equal width, depth and active feed-forward width (sizes: fine, coarse)")
+    ap.add_argument("--gulisun-models", default="gulisun,suvazen", help="which decoders --gulisun runs")
     ap.add_argument("--decode-steps", type=int, default=32)
     ap.add_argument("--eager", action="store_true",
                     help="decoders launch their kernels one by one instead of replaying a captured HIP graph (for "
@@ -572,6 +675,11 @@ def main():
         legs = suvazen_leg(dev, args.suvazen.split(","), models=args.suvazen_models.split(","), eager=args.eager)
         dev.close()
         print(json.dumps({"metric": "Suvazen prefill and decode beside Llama", "data": "synthetic", "n_gpus": 1, "legs": legs}))
+        return
+    if args.gulisun:
+        legs = gulisun_leg(dev, args.gulisun.split(","), models=args.gulisun_models.split(","), eager=args.eager)
+        dev.close()
+        print(json.dumps({"metric": "Gulisun prefill and decode beside Suvazen", "data": "synthetic", "n_gpus": 1, "legs": legs}))
         return
     fmt, rows, cols = synth.Q4_K, 4096, 11008
     alg = algorithmic_bytes(fmt, rows, cols)
