@@ -377,71 +377,78 @@ __global__ __launch_bounds__(256) void k_latent_query(const LatentArgs a, const 
             put(a.kv_p + j, c * turned(a, j, (size_t)*pos_ptr, [&](int i) { return qh[a.dim + i]; }));
 }
 
-// grid (ceil(heads / 16), splits), 2 wavefronts that each take 32 positions of a 64-position tile with all 16 heads,
-// tiles dealt to the splits round robin.  Rows come from memory straight into the first product's operand and, once
-// more, through LDS (transposed, in the key order the second product gets its weights in).  NT: kv_p / 16 at most.
+// grid (ceil(heads / 16), splits), tiles of 32 positions dealt to the splits round robin.  The tile's rows go to LDS
+// once.  The 4 wavefronts share the first product's K (their sums meet in LDS), repeat the softmax over the tile's 32
+// positions, and each take a quarter of the latent's columns in the second product, whose K index 8 g + e stands for key
+// 4 g + e of the tile's first 16 (e < 4) or of the others.  NT: kv_p / 16 at most.
 template <int NT>
-__global__ __launch_bounds__(128) void k_latent_decode(const bf16 *__restrict__ qa, const bf16 *__restrict__ cache,
+__global__ __launch_bounds__(256) void k_latent_decode(const bf16 *__restrict__ qa, const bf16 *__restrict__ cache,
                                                        const int *__restrict__ pos_ptr, float *__restrict__ part, int H, int row, int kv_p,
                                                        int n_splits) {
-    constexpr int NKS = NT / 2 + 4, VP = 40;
-    __shared__ __align__(16) bf16 s_v[2][NT * 16 * VP];
-    __shared__ float s_m[16], s_l[16];
-    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    constexpr int KT = 32, WIDTH = NT * 16 + 128, NKS = (WIDTH / 32 + 3) / 4, P = WIDTH + 8, LOADS = KT * WIDTH / 8 / 256, ND = NT / 4;
+    __shared__ __align__(16) bf16 tile[KT * P];
+    __shared__ __align__(16) f32x4 sums[4][2][64];
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int r16 = lane & 15, g = lane >> 4;
-    const int h = blockIdx.x * 16 + r16, split = blockIdx.y, nks = row >> 5;
+    const int h = blockIdx.x * 16 + r16, split = blockIdx.y, nks = row >> 5, chunks = row >> 3;
     const bf16 *q0 = qa + (size_t)min(h, H - 1) * row + g * 8, *q1 = q0 + (size_t)H * row;
     bf16x8 qh[NKS], ql[NKS];
 #pragma unroll
-    for (int ks = 0; ks < NKS; ++ks)
-        if (ks < nks) {
-            qh[ks] = *(const bf16x8 *)(q0 + ks * 32);
-            ql[ks] = *(const bf16x8 *)(q1 + ks * 32);
-        }
+    for (int i = 0; i < NKS; ++i) {
+        const int ks = min(wave + 4 * i, nks - 1);
+        qh[i] = *(const bf16x8 *)(q0 + ks * 32);
+        ql[i] = *(const bf16x8 *)(q1 + ks * 32);
+    }
     const int pos = *pos_ptr;
-    float m = LOW, l = 0.0f;
-    f32x4 o[NT];
+    u32x4v reg[LOADS];
+    auto request = [&](int p0) __attribute__((always_inline)) {
 #pragma unroll
-    for (int d = 0; d < NT; ++d) o[d] = f32x4{0.f, 0.f, 0.f, 0.f};
-    bf16 *sv = s_v[wave];
-    for (int p0 = split * 64 + wave * 32; p0 <= pos; p0 += n_splits * 64) {
+        for (int i = 0; i < LOADS; ++i) {
+            const int e = tid + i * 256, k = e / chunks;
+            if (k < KT) reg[i] = *(const u32x4v *)(cache + (size_t)min(p0 + k, pos) * row + (e - k * chunks) * 8);
+        }
+    };
+    float m = LOW, l = 0.0f;
+    f32x4 o[ND];
+#pragma unroll
+    for (int d = 0; d < ND; ++d) o[d] = f32x4{0.f, 0.f, 0.f, 0.f};
+    const int step = n_splits * KT;
+    if (split * KT <= pos) request(split * KT);
+    for (int p0 = split * KT; p0 <= pos; p0 += step) {
+#pragma unroll
+        for (int i = 0; i < LOADS; ++i) {
+            const int e = tid + i * 256, k = e / chunks;
+            if (k < KT) *(u32x4v *)&tile[k * P + (e - k * chunks) * 8] = reg[i];
+        }
+        __syncthreads();
+        if (p0 + step <= pos) request(p0 + step);
         f32x4 s[2];
 #pragma unroll
-        for (int kt = 0; kt < 2; ++kt) {
-            const bf16 *k = cache + (size_t)min(p0 + kt * 16 + r16, pos) * row + g * 8;
-            s[kt] = f32x4{0.f, 0.f, 0.f, 0.f};
+        for (int kt = 0; kt < 2; ++kt) s[kt] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-            for (int ks = 0; ks < NKS; ++ks)
-                if (ks < nks) {
-                    const bf16x8 kf = *(const bf16x8 *)(k + ks * 32);
-                    s[kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, ql[ks], s[kt], 0, 0, 0);
-                    s[kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qh[ks], s[kt], 0, 0, 0);
-                }
-        }
-        {   // lane: keys 2 r16 and 2 r16 + 1, chunks g, g + 4, ... of eight values
-            const bf16 *v0 = cache + (size_t)min(p0 + 2 * r16, pos) * row, *v1 = cache + (size_t)min(p0 + 2 * r16 + 1, pos) * row;
-            const int k = 2 * r16, at = ((k >> 2) & 3) * 8 + (k >> 4) * 4 + (k & 3);
+        for (int i = 0; i < NKS; ++i) {
+            const int ks = wave + 4 * i;
+            if (ks >= nks) break;
 #pragma unroll
-            for (int it = 0; it < NT / 2; ++it) {
-                const int c = (g + it * 4) * 8;
-                if (c >= kv_p) continue;
-                const u32x4v a0 = *(const u32x4v *)(v0 + c), a1 = *(const u32x4v *)(v1 + c);
-#pragma unroll
-                for (int j = 0; j < 8; ++j) {
-                    const uint32_t w0 = a0[j >> 1], w1 = a1[j >> 1];
-                    const uint32_t lo = j & 1 ? w0 >> 16 : w0 & 0xFFFFu, hi = j & 1 ? w1 & 0xFFFF0000u : w1 << 16;
-                    *(uint32_t *)&sv[(c + j) * VP + at] = lo | hi;
-                }
+            for (int kt = 0; kt < 2; ++kt) {
+                const bf16x8 kf = *(const bf16x8 *)&tile[(kt * 16 + r16) * P + ks * 32 + g * 8];
+                s[kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, ql[i], s[kt], 0, 0, 0);
+                s[kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qh[i], s[kt], 0, 0, 0);
             }
         }
+#pragma unroll
+        for (int kt = 0; kt < 2; ++kt) sums[wave][kt][lane] = s[kt];
+        __syncthreads();
         float mx = MASKED;
 #pragma unroll
-        for (int kt = 0; kt < 2; ++kt)
+        for (int kt = 0; kt < 2; ++kt) {
+            s[kt] = (sums[0][kt][lane] + sums[1][kt][lane]) + (sums[2][kt][lane] + sums[3][kt][lane]);
 #pragma unroll
             for (int j = 0; j < 4; ++j) {
                 if (p0 + kt * 16 + 4 * g + j > pos) s[kt][j] = MASKED;
                 mx = fmaxf(mx, s[kt][j]);
             }
+        }
         mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
         mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
         const float m_new = fmaxf(m, mx), corr = __builtin_amdgcn_exp2f(m - m_new);
@@ -456,37 +463,31 @@ __global__ __launch_bounds__(128) void k_latent_decode(const bf16 *__restrict__ 
             lo[e] = (bf16)(w - (float)hi[e]);
         }
         l = l * corr + sum;
-        __builtin_amdgcn_wave_barrier();
 #pragma unroll
-        for (int d = 0; d < NT; ++d) {
-            if (d * 16 >= kv_p) continue;
-            const bf16x8 vt = *(const bf16x8 *)&sv[(d * 16 + r16) * VP + g * 8];
+        for (int d = 0; d < ND; ++d) {
+            const int c = (wave + 4 * d) * 16;
+            if (c >= kv_p) break;
+            bf16x8 vt;
+#pragma unroll
+            for (int e = 0; e < 8; ++e) vt[e] = tile[((e >> 2) * 16 + 4 * g + (e & 3)) * P + c + r16];
             o[d] *= corr;
             o[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vt, lo, o[d], 0, 0, 0);
             o[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vt, hi, o[d], 0, 0, 0);
         }
-        __builtin_amdgcn_wave_barrier();
+        __syncthreads();  // the tile and the sums are consumed
     }
     l += __shfl_xor(l, 16, 64);
     l += __shfl_xor(l, 32, 64);
-    // the second wavefront's sums through its own part of LDS
-    f32x4 *so = (f32x4 *)s_v[1];   // [NT][64 lanes]: 1024 bytes of the 1280 per tile
-    if (wave == 1) {
-#pragma unroll
-        for (int d = 0; d < NT; ++d)
-            if (d * 16 < kv_p) so[d * 64 + lane] = o[d];
-        if (g == 0) { s_m[r16] = m; s_l[r16] = l; }
-    }
-    __syncthreads();
-    if (wave == 1 || h >= H) return;
-    const float mm = fmaxf(m, s_m[r16]), f0 = __builtin_amdgcn_exp2f(m - mm), f1 = __builtin_amdgcn_exp2f(s_m[r16] - mm);
+    if (h >= H) return;
     float *p = part + ((size_t)h * n_splits + split) * (kv_p + 4);
 #pragma unroll
-    for (int d = 0; d < NT; ++d)
-        if (d * 16 < kv_p) *(f32x4 *)(p + d * 16 + 4 * g) = o[d] * f0 + so[d * 64 + lane] * f1;
-    if (g == 0) {
-        p[kv_p] = mm;
-        p[kv_p + 1] = l * f0 + s_l[r16] * f1;
+    for (int d = 0; d < ND; ++d) {
+        const int c = (wave + 4 * d) * 16;
+        if (c < kv_p) *(f32x4 *)(p + c + 4 * g) = o[d];
+    }
+    if (wave == 0 && g == 0) {
+        p[kv_p] = m;
+        p[kv_p + 1] = l;
     }
 }
 
@@ -537,15 +538,25 @@ __global__ __launch_bounds__(256) void k_latent_merge(const LatentArgs a, const 
         ls = p[(size_t)lane * pitch + a.kv_p + 1];
     }
     const float sink = a.sink ? a.sink[h] * LOG2E : MASKED;
+    const int sg = tid / C4, c4 = tid % C4;   // thread: splits sg, sg + SG, ... of four columns
+    constexpr int FRONT = 16;
+    f32x4 v[FRONT];
+#pragma unroll
+    for (int j = 0; j < FRONT; ++j) v[j] = *(const f32x4 *)(p + (size_t)min(sg + SG * j, n_splits - 1) * pitch + 4 * c4);
+    __builtin_amdgcn_sched_barrier(0);  // every load above is requested before anything below waits
     const float m = fmaxf(wave_max(ms), sink);
     const float e = lane < n_splits ? __builtin_amdgcn_exp2f(ms - m) : 0.0f;
     const float f = e / (wave_sum(ls * e) + (a.sink ? __builtin_amdgcn_exp2f(sink - m) : 0.0f));
     if (wave == 0) factor[lane] = f;
     __syncthreads();
-    const int sg = tid / C4, c4 = tid % C4;   // thread: splits sg, sg + SG, ... of four columns
     f32x4 o{0.f, 0.f, 0.f, 0.f};
-    if (sg < SG)
-        for (int s = sg; s < n_splits; s += SG) o += *(const f32x4 *)(p + (size_t)s * pitch + 4 * c4) * factor[s];
+    if (sg < SG) {
+#pragma unroll
+        for (int j = 0; j < FRONT; ++j)
+            if (sg + SG * j < n_splits) o += v[j] * factor[sg + SG * j];
+#pragma unroll 8
+        for (int s = sg + SG * FRONT; s < n_splits; s += SG) o += *(const f32x4 *)(p + (size_t)s * pitch + 4 * c4) * factor[s];
+    }
     red[tid] = o;
     __syncthreads();
     if (tid < C4) {
@@ -608,7 +619,7 @@ static int decode_tiles(const candy_hip_latent_spec &s) {
 
 int latent_splits(const candy_hip_device *dev, const candy_hip_latent_spec &s, int max_pos) {
     const int64_t heads = (s.n_heads + 15) / 16;
-    return (int)std::max<int64_t>(1, std::min<int64_t>({64, (max_pos + 63) / 64, 2 * (int64_t)dev->num_cus / heads}));
+    return (int)std::max<int64_t>(1, std::min<int64_t>({64, (max_pos + 31) / 32, 2 * (int64_t)dev->num_cus / heads}));
 }
 size_t latent_query_bytes(const candy_hip_latent_spec &s) { return (size_t)s.n_heads * latent_row(s) * 4; }
 size_t latent_scratch_floats(const candy_hip_latent_spec &s, int n_splits) {
@@ -744,7 +755,7 @@ int launch_latent_decode(candy_hip_device *dev, const LatentAttn &A, const int *
     else decode_query<bf16, false>(dev, A, a, pos_ptr);
     CANDY_LAUNCH_CHECK();
     if (nt) {
-        const dim3 g((unsigned)((a.H + 15) / 16), (unsigned)A.n_splits), b(128);
+        const dim3 g((unsigned)((a.H + 15) / 16), (unsigned)A.n_splits), b(256);
 #define CANDY_LD(NT)                                                                                                                \
     case NT:                                                                                                                        \
         hipLaunchKernelGGL((k_latent_decode<NT>), g, b, 0, dev->stream, (const bf16 *)A.qa, (const bf16 *)A.cache, pos_ptr, A.part,  \

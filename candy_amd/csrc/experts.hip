@@ -31,6 +31,7 @@ __device__ __forceinline__ void choose(const float *z, int E, int top, int *ids,
         const int e = e0 + lane;
         const float mine = e < E ? z[e] : 0.0f;
         int rank = 0;
+#pragma unroll 8
         for (int f = 0; f < E; ++f) rank += z[f] > mine || (z[f] == mine && f < e);
         if (e < E && rank < top) {
             const float s = expf(mine - mx) / sum;
@@ -45,59 +46,82 @@ __device__ __forceinline__ void choose(const float *z, int E, int top, int *ids,
 }
 
 // ------------------------------------------------------------------ prompts
-constexpr int ROUTE_T = 16;
-// grid ceil(n / 16), 4 wavefronts that share K; 64 experts per round
-__global__ __launch_bounds__(256) void k_route(const float *__restrict__ x, int64_t ldx, const bf16 *__restrict__ W, int ld, int E, int top,
-                                               int n, int *__restrict__ ids, float *__restrict__ weights) {
-    extern __shared__ __align__(16) float z[];        // [16][E] scores, then [4][64][17] sums of the wavefronts
+constexpr int ROUTE_T = 16, ROUTE_W = 8, ROUTE_U = 4;   // tokens and wavefronts of a workgroup, K steps requested together
+// grid ceil(n / 16), 8 wavefronts that share K; 64 experts per round
+__global__ __launch_bounds__(64 * ROUTE_W) void k_route(const float *__restrict__ x, int64_t ldx, const bf16 *__restrict__ W, int ld, int E,
+                                                        int top, int n, int *__restrict__ ids, float *__restrict__ weights) {
+    extern __shared__ __align__(16) float z[];        // [16][E] scores, then [4][64][17] sums of pairs of wavefronts
     const int Ep = E | 1;                              // odd pitch
     float *red = z + ROUTE_T * Ep;
     int *s_ids = (int *)red;                           // once the scores stand: [16][top], [16][top]
     float *s_w = red + ROUTE_T * top;
-    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r16 = lane & 15, g = lane >> 4;
-    const int t0 = blockIdx.x * ROUTE_T;
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), r16 = lane & 15, g = lane >> 4;
+    const int t0 = blockIdx.x * ROUTE_T, steps = ld >> 5;
     const float *xr = x + (size_t)min(t0 + r16, n - 1) * ldx + g * 8;
     for (int e0 = 0; e0 < E; e0 += 64) {
         f32x4 acc[4];
 #pragma unroll
         for (int i = 0; i < 4; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
         const bf16 *w = W + (size_t)(e0 + r16) * ld + g * 8;
-#pragma unroll 2
-        for (int k = wave * 32; k < ld; k += 128) {
-            float f[8];
-            lds8(xr + k, f);
-            bf16x8 part[3];
+        const int strips = min(4, (E - e0 + 15) >> 4);
+        for (int s0 = wave; s0 < steps; s0 += ROUTE_W * ROUTE_U) {
+            f32x4 xv[ROUTE_U][2];
+            bf16x8 wv[ROUTE_U][4];
 #pragma unroll
-            for (int j = 0; j < 8; ++j) {
-                part[0][j] = (bf16)f[j];
-                const float r1 = f[j] - (float)part[0][j];
-                part[1][j] = (bf16)r1;
-                part[2][j] = (bf16)(r1 - (float)part[1][j]);
+            for (int u = 0; u < ROUTE_U; ++u) {
+                const int k = min(s0 + u * ROUTE_W, steps - 1) * 32;
+                xv[u][0] = *(const f32x4 *)(xr + k);
+                xv[u][1] = *(const f32x4 *)(xr + k + 4);
+#pragma unroll
+                for (int i = 0; i < 4; ++i)
+                    if (i < strips) wv[u][i] = *(const bf16x8 *)(w + (size_t)i * 16 * ld + k);
             }
 #pragma unroll
-            for (int i = 0; i < 4; ++i) {
-                const bf16x8 wf = *(const bf16x8 *)(w + (size_t)i * 16 * ld + k);
+            for (int u = 0; u < ROUTE_U; ++u) {
+                if (s0 + u * ROUTE_W >= steps) break;
+                bf16x8 part[3];
 #pragma unroll
-                for (int p = 2; p >= 0; --p) acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf, part[p], acc[i], 0, 0, 0);
+                for (int j = 0; j < 8; ++j) {
+                    const float f = xv[u][j >> 2][j & 3];
+                    part[0][j] = (bf16)f;
+                    const float r1 = f - (float)part[0][j];
+                    part[1][j] = (bf16)r1;
+                    part[2][j] = (bf16)(r1 - (float)part[1][j]);
+                }
+#pragma unroll
+                for (int i = 0; i < 4; ++i)
+                    if (i < strips) {
+#pragma unroll
+                        for (int p = 2; p >= 0; --p) acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wv[u][i], part[p], acc[i], 0, 0, 0);
+                    }
             }
         }
         // lane: token r16, experts e0 + 16 i + 4 g + j
+        for (int half = 1; half >= 0; --half) {   // the second four wavefronts' sums, then the first four's on top
+            if (wave >> 2 == half) {
 #pragma unroll
-        for (int i = 0; i < 4; ++i)
+                for (int i = 0; i < 4; ++i)
 #pragma unroll
-            for (int j = 0; j < 4; ++j) red[(wave * 64 + i * 16 + 4 * g + j) * 17 + r16] = acc[i][j];
-        __syncthreads();
-        for (int i = tid; i < 64 * ROUTE_T; i += 256) {
+                    for (int j = 0; j < 4; ++j) {
+                        float *s = &red[((wave & 3) * 64 + i * 16 + 4 * g + j) * 17 + r16];
+                        *s = half ? acc[i][j] : *s + acc[i][j];
+                    }
+            }
+            __syncthreads();
+        }
+        for (int i = tid; i < 64 * ROUTE_T; i += 64 * ROUTE_W) {
             const int t = i & 15, e = i >> 4;
-            if (e0 + e < E)
-                z[t * Ep + e0 + e] =
-                    ordered((red[e * 17 + t] + red[(64 + e) * 17 + t]) + (red[(128 + e) * 17 + t] + red[(192 + e) * 17 + t]));
+            if (e0 + e >= E) continue;
+            float sum = 0.0f;
+#pragma unroll
+            for (int v = 0; v < ROUTE_W / 2; ++v) sum += red[(v * 64 + e) * 17 + t];
+            z[t * Ep + e0 + e] = ordered(sum);
         }
         __syncthreads();
     }
-    for (int t = wave; t < ROUTE_T; t += 4) choose(z + t * Ep, E, top, s_ids + t * top, s_w + t * top);
+    for (int t = wave; t < ROUTE_T; t += ROUTE_W) choose(z + t * Ep, E, top, s_ids + t * top, s_w + t * top);
     __syncthreads();
-    for (int i = tid; i < ROUTE_T * top; i += 256)
+    for (int i = tid; i < ROUTE_T * top; i += 64 * ROUTE_W)
         if (t0 + i / top < n) {
             ids[(size_t)t0 * top + i] = s_ids[i];
             weights[(size_t)t0 * top + i] = s_w[i];
@@ -112,7 +136,15 @@ __global__ __launch_bounds__(1024) void k_deal(const int *__restrict__ ids, int 
     const int tid = threadIdx.x;
     members[tid] = 0;
     __syncthreads();
-    for (int i = tid; i < count; i += 1024) atomicAdd(&members[ids[i]], 1);
+    constexpr int AHEAD = 4;
+    for (int i0 = tid; i0 < count; i0 += 1024 * AHEAD) {
+        int e[AHEAD];
+#pragma unroll
+        for (int k = 0; k < AHEAD; ++k) e[k] = ids[min(i0 + 1024 * k, count - 1)];
+#pragma unroll
+        for (int k = 0; k < AHEAD; ++k)
+            if (i0 + 1024 * k < count) atomicAdd(&members[e[k]], 1);
+    }
     __syncthreads();
     const int mine = members[tid], my_tiles = (mine + rows - 1) / rows;
     int cur = 0;
@@ -130,7 +162,14 @@ __global__ __launch_bounds__(1024) void k_deal(const int *__restrict__ ids, int 
     if (tid == MAX_EXPERTS - 1) *n_tiles = tile_end[cur][tid];
     members[tid] = begin;
     __syncthreads();
-    for (int i = tid; i < count; i += 1024) perm[atomicAdd(&members[ids[i]], 1)] = i;
+    for (int i0 = tid; i0 < count; i0 += 1024 * AHEAD) {
+        int e[AHEAD];
+#pragma unroll
+        for (int k = 0; k < AHEAD; ++k) e[k] = ids[min(i0 + 1024 * k, count - 1)];
+#pragma unroll
+        for (int k = 0; k < AHEAD; ++k)
+            if (i0 + 1024 * k < count) perm[atomicAdd(&members[e[k]], 1)] = i0 + 1024 * k;
+    }
 }
 
 // ------------------------------------------------------------------ decode
@@ -274,7 +313,7 @@ static size_t down_lds(const candy_hip_expert_spec &s, size_t es) {
     return chunks * 8 + ((chunks + 3) & ~(size_t)3) * 4 + K * es;
 }
 static size_t route_lds(const candy_hip_expert_spec &s) {
-    return ((size_t)ROUTE_T * (s.n_experts | 1) + std::max<size_t>(4 * 64 * 17, 2 * ROUTE_T * (size_t)s.top)) * 4;
+    return ((size_t)ROUTE_T * (s.n_experts | 1) + std::max<size_t>(ROUTE_W / 2 * 64 * 17, 2 * ROUTE_T * (size_t)s.top)) * 4;
 }
 
 int check_expert_spec(const candy_hip_expert_spec &s, int d) {
@@ -302,7 +341,7 @@ size_t expert_list_ints(const candy_hip_expert_spec &s, int n) { return deal_per
 int launch_experts_prompt(candy_hip_device *dev, const ExpertLayer &A, int n) {
     const candy_hip_expert_spec &s = A.s;
     const int rows = deal_rows(s, n, A.f32);
-    hipLaunchKernelGGL(k_route, dim3((unsigned)((n + ROUTE_T - 1) / ROUTE_T)), dim3(256), route_lds(s), dev->stream, A.x, A.ldx,
+    hipLaunchKernelGGL(k_route, dim3((unsigned)((n + ROUTE_T - 1) / ROUTE_T)), dim3(64 * ROUTE_W), route_lds(s), dev->stream, A.x, A.ldx,
                        (const bf16 *)A.w.router->data, (int)A.w.router->ld, s.n_experts, s.top, n, A.ids, A.weights);
     CANDY_LAUNCH_CHECK();
     int *n_tiles = A.list, *perm = A.list + 4;

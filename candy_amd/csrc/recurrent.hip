@@ -52,30 +52,50 @@ __device__ __forceinline__ int gate_column(const LruArgs &a, int block, int off)
 }
 
 // ------------------------------------------------------------------ prompts
-constexpr int CONV_T = 4;
+constexpr int CONV_T = 8, CONV_TAPS = 4;
 
-// grid (blocks * size_p / 256, ceil(n / 4)): one thread per padded channel and four tokens
-template <class AT>
+// The input of the convolution for token t of the portion (t < 0: earlier ones), bias included.
+__device__ __forceinline__ float conv_input(const LruArgs &a, const Partial &z, const float *history, int c, float bx, int t, int pos0) {
+    if (t >= 0) return z_at(z, (size_t)t, a.wp + c) + bx;
+    return pos0 + t >= 0 ? history[(size_t)((pos0 + t) % a.taps) * a.wp + c] : 0.0f;
+}
+
+// grid (blocks * size_p / 256, ceil(n / 8)): one thread per padded channel and eight tokens.  FEW: at most 4 taps, the
+// inputs are requested together.
+template <class AT, bool FEW>
 __global__ __launch_bounds__(256) void k_lru_conv(const LruArgs a, const Partial z, const float *__restrict__ history, AT *__restrict__ u,
                                                   int n, int pos0) {
     const int cp = blockIdx.x * 256 + threadIdx.x, cols = a.blocks * a.size_p;
     if (cp >= cols) return;
     const int off = cp % a.size_p, c = cp / a.size_p * a.size + off, t0 = blockIdx.y * CONV_T;
-    const bool real = off < a.size;
     float acc[CONV_T];
 #pragma unroll
-    for (int k = 0; k < CONV_T; ++k) acc[k] = real ? a.p.conv_b[c] : 0.0f;
-    if (real) {
-        const float bx = a.p.bx[c];
-        for (int t = t0 - a.taps + 1; t < t0 + CONV_T; ++t) {
-            if (t >= n) break;
-            float v = 0.0f;
-            if (t >= 0) v = z_at(z, (size_t)t, a.wp + c) + bx;
-            else if (pos0 + t >= 0) v = history[(size_t)((pos0 + t) % a.taps) * a.wp + c];
+    for (int k = 0; k < CONV_T; ++k) acc[k] = 0.0f;
+    if (off < a.size) {
+        const float bx = a.p.bx[c], cb = a.p.conv_b[c];
 #pragma unroll
-            for (int k = 0; k < CONV_T; ++k) {
-                const int tap = t - (t0 + k) + a.taps - 1;
-                if (tap >= 0 && tap < a.taps) acc[k] = fmaf(a.p.conv[(size_t)tap * a.wp + c], v, acc[k]);
+        for (int k = 0; k < CONV_T; ++k) acc[k] = cb;
+        if (FEW) {
+            float v[CONV_T + CONV_TAPS - 1], w[CONV_TAPS];
+#pragma unroll
+            for (int j = 0; j < CONV_TAPS; ++j) w[j] = j < a.taps ? a.p.conv[(size_t)(a.taps - 1 - j) * a.wp + c] : 0.0f;  // j tokens back
+#pragma unroll
+            for (int i = 0; i < CONV_T + CONV_TAPS - 1; ++i) {
+                const int t = min(t0 + i - (CONV_TAPS - 1), n - 1);
+                v[i] = CONV_TAPS - 1 - i < a.taps ? conv_input(a, z, history, c, bx, t, pos0) : 0.0f;  // what no tap reaches may not exist
+            }
+#pragma unroll
+            for (int k = 0; k < CONV_T; ++k)
+#pragma unroll
+                for (int j = CONV_TAPS - 1; j >= 0; --j) acc[k] = fmaf(w[j], v[k + CONV_TAPS - 1 - j], acc[k]);
+        } else {
+            for (int t = t0 - a.taps + 1; t < t0 + CONV_T && t < n; ++t) {
+                const float v = conv_input(a, z, history, c, bx, t, pos0);
+#pragma unroll
+                for (int k = 0; k < CONV_T; ++k) {
+                    const int tap = t - (t0 + k) + a.taps - 1;
+                    if (tap >= 0 && tap < a.taps) acc[k] = fmaf(a.p.conv[(size_t)tap * a.wp + c], v, acc[k]);
+                }
             }
         }
     }
@@ -86,28 +106,34 @@ __global__ __launch_bounds__(256) void k_lru_conv(const LruArgs a, const Partial
 
 constexpr int SCAN_U = 8;   // tokens whose values are requested together
 
-// f(t, a, b) over tokens t0 .. t1 - 1 of channel c
-template <class AT, class F>
-__device__ __forceinline__ void lru_tokens(const LruArgs &a, const float *__restrict__ g, const AT *__restrict__ u, int c, int t0, int t1, F f) {
+// f(t, a, b, y) over tokens t0 .. t1 - 1 of channel c; Y: y is the projection for the other branch
+template <bool Y, class AT, class F>
+__device__ __forceinline__ void lru_tokens(const LruArgs &a, const Partial &z, const float *__restrict__ g, const AT *__restrict__ u, int c,
+                                           int t0, int t1, F f) {
     const int block = c / a.size, off = c - block * a.size, gld = 2 * a.blocks * a.size_p, uld = a.blocks * a.size_p;
     const float *gr = g + gate_column(a, block, off);
     const AT *uc = u + block * a.size_p + off;
     const float rate = decay_rate(a.p.lam[c]), br = a.p.ra_b[c], bi = a.p.ri_b[c];
     for (int t = t0; t < t1; t += SCAN_U) {
-        float r[SCAN_U], i[SCAN_U], x[SCAN_U];
+        float r[SCAN_U], i[SCAN_U], x[SCAN_U], y[SCAN_U];
 #pragma unroll
         for (int k = 0; k < SCAN_U; ++k) {
             const size_t tt = (size_t)min(t + k, t1 - 1);
             r[k] = gr[tt * gld];
             i[k] = gr[tt * gld + 64];
             x[k] = (float)uc[tt * uld];
+            y[k] = Y ? z.p[tt * z.ld + c] : 0.0f;
+        }
+        for (int q = 1; Y && q < z.copies; ++q) {
+#pragma unroll
+            for (int k = 0; k < SCAN_U; ++k) y[k] += z.p[(size_t)q * z.stride + (size_t)min(t + k, t1 - 1) * z.ld + c];
         }
 #pragma unroll
         for (int k = 0; k < SCAN_U; ++k)
             if (t + k < t1) {
                 float aa, bb;
                 lru_coefficients(r[k] + br, i[k] + bi, x[k], rate, aa, bb);
-                f(t + k, aa, bb);
+                f(t + k, aa, bb, y[k]);
             }
     }
 }
@@ -121,7 +147,7 @@ __global__ __launch_bounds__(256) void k_lru_chunks(const LruArgs a, const float
     if (blockIdx.y == 0) scan[c] = fresh ? 0.0f : state[c];
     float A = 1.0f, B = 0.0f;
     const int t0 = blockIdx.y * chunk;
-    lru_tokens(a, g, u, c, t0, min(t0 + chunk, n), [&](int, float aa, float bb) {
+    lru_tokens<false>(a, Partial{}, g, u, c, t0, min(t0 + chunk, n), [&](int, float aa, float bb, float) {
         A *= aa;
         B = fmaf(aa, B, bb);
     });
@@ -142,12 +168,12 @@ __global__ __launch_bounds__(256) void k_lru_apply(const LruArgs a, const Partia
     }
     float S = scan[c];
     const float *s = scan + a.wp + c;
-#pragma unroll 4
+#pragma unroll 8
     for (int k = 0; k < (int)blockIdx.y; ++k, s += 2 * (size_t)a.wp) S = fmaf(s[0], S, s[a.wp]);
     const float by = a.p.by[c];
-    lru_tokens(a, g, u, c, t0, t1, [&](int t, float aa, float bb) {
+    lru_tokens<true>(a, z, g, u, c, t0, t1, [&](int t, float aa, float bb, float y) {
         S = fmaf(aa, S, bb);
-        out[(size_t)t * a.ldo + c] = (AT)(S * gelu_tanh_f(z_at(z, (size_t)t, c) + by));
+        out[(size_t)t * a.ldo + c] = (AT)(S * gelu_tanh_f(y + by));
     });
     if (t1 < n) return;
     state[c] = S;
@@ -248,8 +274,11 @@ static int lru_prompt(candy_hip_device *dev, const LruLayer &A, int n, int pos0)
     const int cols = a.blocks * a.size_p;
     CANDY_REQUIRE(A.gates->rows == 2 * cols && A.gates->ld == a.size_p && a.out_cols <= a.wp && (n + CONV_T - 1) / CONV_T <= 65535,
                   "internal: recurrent launch");
-    hipLaunchKernelGGL((k_lru_conv<AT>), dim3((unsigned)((cols + 255) / 256), (unsigned)((n + CONV_T - 1) / CONV_T)), dim3(256), 0, dev->stream,
-                       a, A.z, A.state + a.wp, (AT *)A.u, n, pos0);
+    const dim3 gc((unsigned)((cols + 255) / 256), (unsigned)((n + CONV_T - 1) / CONV_T));
+    if (a.taps <= CONV_TAPS)
+        hipLaunchKernelGGL((k_lru_conv<AT, true>), gc, dim3(256), 0, dev->stream, a, A.z, A.state + a.wp, (AT *)A.u, n, pos0);
+    else
+        hipLaunchKernelGGL((k_lru_conv<AT, false>), gc, dim3(256), 0, dev->stream, a, A.z, A.state + a.wp, (AT *)A.u, n, pos0);
     CANDY_LAUNCH_CHECK();
     DenseLaunch D;
     D.w = A.gates; D.x = A.u; D.ldx = cols; D.f32 = A.f32; D.m = n; D.block_rows = 2 * a.size_p;

@@ -36,6 +36,11 @@ def rel(got, want):
     return float(np.sqrt(((got - want) ** 2).mean(1)).max() / (np.sqrt((want ** 2).mean()) + 1e-30))
 
 
+def own(got, want):
+    """Worst row: root mean square of the difference over that of the row itself."""
+    return max(rel(g, w) for g, w in zip(got, want))
+
+
 def up(n, to):
     return -(-n // to) * to
 
@@ -368,9 +373,9 @@ def test_experts(dev, d, experts, top, ff, shared, act):
     for n in (200, 2, 65, 1):
         got, gids, gw = dev.experts(case.spec, act, case.dense, x[:n])
         assert np.array_equal(gids, ids[:n]) and np.abs(gw - weights[:n]).max() < 2e-5
-        assert rel(got, want[:n]) < tol, n
+        assert own(got, want[:n]) < tol, n
     rows = np.concatenate([dev.experts(case.spec, act, case.dense, x[t:t + 1], decode=True) for t in range(12)])
-    assert rel(rows, want[:12]) < tol
+    assert own(rows, want[:12]) < tol
 
 
 @pytest.mark.parametrize("act", ACTS)
