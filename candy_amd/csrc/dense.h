@@ -76,10 +76,12 @@ struct Partial {
 };
 
 // Activation rows dealt to experts: w holds `expert_rows` rows per expert one after the other; tile t of the list takes
-// rows first .. first + count - 1 of `perm` for one expert.  perm holds slots (token * top + choice); a slot's
+// rows first .. first + count - 1 of `perm` for one expert, whose tiles are of_expert in number from tile0 on.  perm holds slots (token * top + choice); a slot's
 // activations are row slot / x_div, its result is row slot.
-struct GroupTile {
-    int expert, first, count, pad;
+struct alignas(16) GroupTile {
+    int expert, first;
+    int count;
+    uint16_t tile0, of_expert;
 };
 struct GroupedRows {
     const int *perm = nullptr;

@@ -222,11 +222,14 @@ __global__ __launch_bounds__(256, 2) void k_dense_mm(const bf16 *__restrict__ W,
         const int per = total >> 3, full = per << 3;
         if (t < full) t = (t & 7) * per + (t >> 3);
     }
-    const int n0 = (t / m_tiles) * BN;
-    int m0 = (t % m_tiles) * BM;
+    int n0 = (t / m_tiles) * BN, m0 = (t % m_tiles) * BM;
     const int *perm = nullptr;
     if (GROUPED) {
-        const GroupTile tile = gr.tiles[t % m_tiles];
+        // expert by expert; within one, its row tiles of one weight tile are neighbours
+        GroupTile tile = gr.tiles[t / n_tiles];
+        const int local = t - tile.tile0 * n_tiles, nt = local / tile.of_expert;
+        n0 = nt * BN;
+        tile = gr.tiles[tile.tile0 + local - nt * tile.of_expert];
         W += (size_t)tile.expert * Np * ld;
         perm = gr.perm + tile.first;
         M = tile.count;

@@ -158,7 +158,7 @@ __global__ __launch_bounds__(1024) void k_deal(const int *__restrict__ ids, int 
         __syncthreads();
     }
     const int begin = end[cur][tid] - mine, tile0 = tile_end[cur][tid] - my_tiles;
-    for (int k = 0; k < my_tiles; ++k) tiles[tile0 + k] = GroupTile{tid, begin + k * rows, min(rows, mine - k * rows), 0};
+    for (int k = 0; k < my_tiles; ++k) tiles[tile0 + k] = GroupTile{tid, begin + k * rows, min(rows, mine - k * rows), (uint16_t)tile0, (uint16_t)my_tiles};
     if (tid == MAX_EXPERTS - 1) *n_tiles = tile_end[cur][tid];
     members[tid] = begin;
     __syncthreads();
