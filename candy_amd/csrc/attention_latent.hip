@@ -408,12 +408,12 @@ __global__ __launch_bounds__(256) void k_latent_decode(const bf16 *__restrict__ 
             if (k < KT) reg[i] = *(const u32x4v *)(cache + (size_t)min(p0 + k, pos) * row + (e - k * chunks) * 8);
         }
     };
+    if (split * KT <= pos) request(split * KT);
     float m = LOW, l = 0.0f;
     f32x4 o[ND];
 #pragma unroll
     for (int d = 0; d < ND; ++d) o[d] = f32x4{0.f, 0.f, 0.f, 0.f};
     const int step = n_splits * KT;
-    if (split * KT <= pos) request(split * KT);
     for (int p0 = split * KT; p0 <= pos; p0 += step) {
 #pragma unroll
         for (int i = 0; i < LOADS; ++i) {
@@ -618,6 +618,7 @@ static int decode_tiles(const candy_hip_latent_spec &s) {
 }
 
 int latent_splits(const candy_hip_device *dev, const candy_hip_latent_spec &s, int max_pos) {
+    if (dev->opt.attn_splits > 0) return dev->opt.attn_splits;  // comparison runs
     const int64_t heads = (s.n_heads + 15) / 16;
     return (int)std::max<int64_t>(1, std::min<int64_t>({64, (max_pos + 31) / 32, 2 * (int64_t)dev->num_cus / heads}));
 }

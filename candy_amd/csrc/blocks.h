@@ -131,10 +131,16 @@ __device__ __forceinline__ float wave_sum(float v) {
     v += dpp_move<0x143, 0xC>(v);  // row_bcast:31 into rows 2 and 3: lane 63 holds the total
     return __int_as_float(__builtin_amdgcn_readlane(__float_as_int(v), 63));
 }
+// Maximum over the 64 lanes of a wavefront; every lane gets it.
 __device__ __forceinline__ float wave_max(float v) {
-#pragma unroll
-    for (int off = 32; off > 0; off >>= 1) v = fmaxf(v, __shfl_xor(v, off, 64));
-    return v;
+    v = fmaxf(v, dpp_move<0xB1>(v));
+    v = fmaxf(v, dpp_move<0x4E>(v));
+    v = fmaxf(v, dpp_move<0x141>(v));
+    v = fmaxf(v, dpp_move<0x140>(v));
+    // rows the broadcast does not reach keep their own value
+    v = fmaxf(v, __int_as_float(__builtin_amdgcn_update_dpp(__float_as_int(v), __float_as_int(v), 0x142, 0xA, 0xF, false)));
+    v = fmaxf(v, __int_as_float(__builtin_amdgcn_update_dpp(__float_as_int(v), __float_as_int(v), 0x143, 0xC, 0xF, false)));
+    return __int_as_float(__builtin_amdgcn_readlane(__float_as_int(v), 63));
 }
 
 

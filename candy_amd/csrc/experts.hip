@@ -17,9 +17,38 @@ namespace candy {
 // a model's numbers have gone wrong.
 __device__ __forceinline__ float ordered(float z) { return z == z ? z : -INFINITY; }
 
-// One wavefront, the scores z[0 .. E) of a token in LDS (ordered()): chosen experts and weights in order of their scores.
+// One wavefront, lane e holding score e of a token's E <= 64 (ordered()): lane k leaves with the k-th choice and its weight.
+__device__ __forceinline__ void choose64(float v, int E, int top, int &id, float &weight) {
+    const int lane = threadIdx.x & 63;
+    uint64_t left = E == 64 ? ~0ull : (1ull << E) - 1;
+    if (lane >= E) v = -INFINITY;
+    float best = wave_max(v), mine = -INFINITY;
+    const float mx = fmaxf(best, LOW), sum = wave_sum(lane < E ? expf(v - mx) : 0.0f);
+    id = 0;
+    for (int k = 0; k < top; ++k) {
+        if (k) best = wave_max(v);
+        const int e = __ffsll((unsigned long long)(__ballot(v == best) & left)) - 1;   // not empty: `left` has top - k members
+        left &= ~(1ull << e);
+        if (lane == k) { id = e; mine = best; }
+        if (lane == e) v = -INFINITY;
+    }
+    const float s = lane < top ? expf(mine - mx) / sum : 0.0f;
+    weight = s / (wave_sum(s) + 1e-20f);
+}
+
+// The same for any number of scores z[0 .. E) in LDS; choices and weights in order of their scores.
 __device__ __forceinline__ void choose(const float *z, int E, int top, int *ids, float *weights) {
     const int lane = threadIdx.x & 63;
+    if (E <= 64) {
+        int id;
+        float w;
+        choose64(lane < E ? z[lane] : 0.0f, E, top, id, w);
+        if (lane < top) {
+            ids[lane] = id;
+            weights[lane] = w;
+        }
+        return;
+    }
     float mx = LOW;
     for (int e = lane; e < E; e += 64) mx = fmaxf(mx, z[e]);
     mx = wave_max(mx);
@@ -180,8 +209,9 @@ struct RowArgs {
 
 constexpr int EXP_U = 4;   // 16-byte requests per row in flight
 
-// Rows of the concatenated up matrices, R per wavefront.  LDS: x, the scores, the choice.
-template <class AT, int R>
+// Rows of the concatenated up matrices, R per wavefront.  FEW: at most 64 experts, every wavefront makes the choice for
+// itself and requests its weights before the activations are staged.  LDS: x; else also the scores and the choice.
+template <class AT, int R, bool FEW>
 __global__ __launch_bounds__(1024) void k_expert_up(const RowArgs a, const float *__restrict__ x, const float *__restrict__ logits,
                                                     AT *__restrict__ act, int *__restrict__ sel) {
     extern __shared__ __align__(16) uint8_t lds[];
@@ -190,24 +220,35 @@ __global__ __launch_bounds__(1024) void k_expert_up(const RowArgs a, const float
     int *ids = (int *)(gate + a.top);
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), threads = blockDim.x;
     const int total = a.top * a.rows_e + a.rows_s, row0 = (blockIdx.x * (threads >> 6) + wave) * R;
-    for (int e = tid; e < a.E; e += threads) z[e] = ordered(logits[e]);
-    typedef AT at4 __attribute__((ext_vector_type(4)));
-    for (int i = tid * 4; i < a.ld; i += threads * 4) *(at4 *)&xs[i] = __builtin_convertvector(*(const f32x4 *)(x + i), at4);
-    __syncthreads();
-    if (wave == 0) {
-        choose(z, a.E, a.top, ids, gate);
-        if (blockIdx.x == 0)
-            for (int k = lane; k < a.top; k += 64) sel[k] = ids[k];
+    int my_id = 0;
+    float my_weight = 0.0f;
+    auto stage = [&]() __attribute__((always_inline)) {
+        typedef AT at4 __attribute__((ext_vector_type(4)));
+        for (int i = tid * 4; i < a.ld; i += threads * 4) *(at4 *)&xs[i] = __builtin_convertvector(*(const f32x4 *)(x + i), at4);
+    };
+    if (FEW) {
+        choose64(ordered(logits[min(lane, a.E - 1)]), a.E, a.top, my_id, my_weight);
+        if (blockIdx.x == 0 && wave == 0 && lane < a.top) sel[lane] = my_id;
+    } else {
+        for (int e = tid; e < a.E; e += threads) z[e] = ordered(logits[e]);
+        stage();
+        __syncthreads();
+        if (wave == 0) {
+            choose(z, a.E, a.top, ids, gate);
+            if (blockIdx.x == 0)
+                for (int k = lane; k < a.top; k += 64) sel[k] = ids[k];
+        }
+        __syncthreads();
     }
-    __syncthreads();
     const bf16 *w[R];
     float scale[R];
 #pragma unroll
     for (int r = 0; r < R; ++r) {
         const int row = min(row0 + r, total - 1), k = row / a.rows_e;
         if (k < a.top) {
-            w[r] = a.W + ((size_t)ids[k] * a.rows_e + (row - k * a.rows_e)) * a.ld;
-            scale[r] = gate[k];
+            const int id = FEW ? __builtin_amdgcn_readlane(my_id, k) : ids[k];
+            w[r] = a.W + ((size_t)id * a.rows_e + (row - k * a.rows_e)) * a.ld;
+            scale[r] = FEW ? __int_as_float(__builtin_amdgcn_readlane(__float_as_int(my_weight), k)) : gate[k];
         } else {
             w[r] = a.shared + (size_t)(row - a.top * a.rows_e) * a.ld;
             scale[r] = 1.0f;
@@ -222,6 +263,10 @@ __global__ __launch_bounds__(1024) void k_expert_up(const RowArgs a, const float
         for (int u = 0; u < EXP_U; ++u)
 #pragma unroll
             for (int r = 0; r < R; ++r) v[r][u] = __builtin_nontemporal_load((const u32x4v *)(w[r] + min(k0 + u * 512 + lane * 8, a.ld - 8)));
+        if (FEW && k0 == 0) {
+            stage();
+            __syncthreads();
+        }
 #pragma unroll
         for (int u = 0; u < EXP_U; ++u) {
             const int k = k0 + u * 512 + lane * 8;
@@ -385,11 +430,17 @@ static int experts_row(candy_hip_device *dev, const ExpertLayer &A) {
     const dim3 gu((unsigned)((total + su.waves * su.rows - 1) / (su.waves * su.rows))), bu((unsigned)(64 * su.waves));
     const size_t lu = up_lds(s, d, sizeof(AT)), ldn = down_lds(s, sizeof(AT));
     CANDY_REQUIRE(lu <= 65536 && ldn <= 163840, "experts too wide for this activation format");
+#define CANDY_UP(R)                                                                                                          \
+    do {                                                                                                                     \
+        if (s.n_experts <= 64) hipLaunchKernelGGL((k_expert_up<AT, R, true>), gu, bu, lu, dev->stream, u, A.x, A.logits, act, A.ids); \
+        else hipLaunchKernelGGL((k_expert_up<AT, R, false>), gu, bu, lu, dev->stream, u, A.x, A.logits, act, A.ids);          \
+    } while (0)
     switch (su.rows) {
-    case 1: hipLaunchKernelGGL((k_expert_up<AT, 1>), gu, bu, lu, dev->stream, u, A.x, A.logits, act, A.ids); break;
-    case 2: hipLaunchKernelGGL((k_expert_up<AT, 2>), gu, bu, lu, dev->stream, u, A.x, A.logits, act, A.ids); break;
-    default: hipLaunchKernelGGL((k_expert_up<AT, 4>), gu, bu, lu, dev->stream, u, A.x, A.logits, act, A.ids); break;
+    case 1: CANDY_UP(1); break;
+    case 2: CANDY_UP(2); break;
+    default: CANDY_UP(4); break;
     }
+#undef CANDY_UP
     CANDY_LAUNCH_CHECK();
     u.W = (const bf16 *)A.w.down->data;
     u.shared = s.shared_ff ? (const bf16 *)A.w.shared_down->data : nullptr;

@@ -284,7 +284,7 @@ static int lru_prompt(candy_hip_device *dev, const LruLayer &A, int n, int pos0)
     D.w = A.gates; D.x = A.u; D.ldx = cols; D.f32 = A.f32; D.m = n; D.block_rows = 2 * a.size_p;
     D.y = A.g; D.ldy = D.n_store = A.gates->rows_pad;
     if (int rc = launch_dense(dev, D)) return rc;
-    const int chunk = std::max(32, (n + MAX_CHUNKS - 1) / MAX_CHUNKS), chunks = (n + chunk - 1) / chunk;
+    const int chunk = std::max(16, (n + MAX_CHUNKS - 1) / MAX_CHUNKS), chunks = (n + chunk - 1) / chunk;
     const dim3 g((unsigned)((a.wp + 255) / 256), (unsigned)chunks);
     hipLaunchKernelGGL((k_lru_chunks<AT>), g, dim3(256), 0, dev->stream, a, A.g, (const AT *)A.u, A.state, A.scan, n, chunk, (int)(pos0 == 0));
     CANDY_LAUNCH_CHECK();
