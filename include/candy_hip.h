@@ -115,7 +115,7 @@ int candy_hip_synchronize(candy_hip_device *dev);       /* device.go:81 Synchron
  *                                         up quantizes them, handing 32-value blocks that two workgroups share through
  *                                         per-block tickets); same bits, measured slower
  *   "attention.splits"           0        comparison runs: decode attention deals the cached positions to this many
- *                                         workgroups per kv head, 1..64 (0: by shape); read when a decoder is created
+ *                                         workgroups per kv head (latent attention: per 16 heads), 1..64 (0: by shape); read when a decoder is created
  *   "prefill.qkv_group"          1        prompt pass: projections that share their input (q / k / v; gate / up) as one
  *                                         grid each where all of them run on the fp16 tiles (0: one launch each)
  *   "prefill.fold_split_sums"    1        prompt pass: the partial copies a projection split along K leaves are summed by the
@@ -488,6 +488,7 @@ int candy_hip_experts(candy_hip_device *dev, const candy_hip_expert_spec *spec, 
 int candy_hip_decoder_free(candy_hip_decoder *m);
 int candy_hip_decoder_set_graph(candy_hip_decoder *m, int enable);
 int candy_hip_decoder_hidden(candy_hip_decoder *m, const float **dev_hidden);
+/* *dev_v is NULL for a model whose cache rows serve as keys and values. */
 int candy_hip_decoder_kv_cache(candy_hip_decoder *m, void **dev_k, void **dev_v, size_t *bytes_each);
 int candy_hip_decoder_decode(candy_hip_decoder *m, int32_t token, int32_t pos, const float **dev_logits,
                              int32_t *next_token);
