@@ -244,7 +244,7 @@ __global__ __launch_bounds__(256, 2) void k_latent_prompt(const LatentArgs a, co
 }
 
 // ------------------------------------------------------------------ one wavefront per (query, head) or (head, split)
-// Softmax over the positions first + 64 i * stride + lane up to pos.  q: this wavefront's query in LDS, in two parts: d1
+// Softmax over the positions p0 .. p0 + 63, p0 = first, first + stride, ..., up to pos.  q: this wavefront's query in LDS, in two parts: d1
 // values against k1 (rows ld1 apart), d2 against k2; values: dv of v.  Lane i holds values i, i + 64, ...
 template <class AT, int NC>
 __device__ __forceinline__ void attend_row(const float *q, const AT *k1, int64_t ld1, int d1, const AT *k2, int64_t ld2, int d2,
